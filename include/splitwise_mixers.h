@@ -10,7 +10,8 @@
  * latent shared by all heads, gated linear attention with a decay per key channel, and the gated residual
  * step of layers that read a mix of all earlier layers' outputs; norms in groups of channels around every
  * sublayer, a causal convolution added to a sublayer's input, the delta rule with one decay per head, attention
- * with sigmoid weights and a softmax router.  A library of its own so that a model that needs only these compiles
+ * with sigmoid weights and a softmax router; latent attention with a query latent, and the stream of decoders that run a
+ * block of layers several times.  A library of its own so that a model that needs only these compiles
  * only these.
  *
  * A step is a RAGGED batch: the new tokens of all sequences back to back in one token dimension.
@@ -36,7 +37,7 @@
 extern "C" {
 #endif
 
-#define SWM_ABI_VERSION 5
+#define SWM_ABI_VERSION 6
 int swm_abi_version(void);
 const char* swm_last_error(void);
 
@@ -167,8 +168,9 @@ int swm_stream_add_norm(float* residual, const void* a, int64_t a_stride, const 
  * out[rows, ff] = g * sigmoid(alpha * g) * (u + shift).  limit may be +inf. */
 int swm_clamped_glu(void* out, const void* in, int64_t in_stride, int64_t rows, int ff, float alpha, float limit,
                     float shift, int act_dtype, void* stream);
-/* out[rows, ff] = max(in, 0)^2 */
-int swm_relu2(void* out, const void* in, int64_t in_stride, int64_t rows, int ff, int act_dtype, void* stream);
+/* out[rows, ff] = max(in, 0)^2, rows out_stride / in_stride elements apart */
+int swm_relu2(void* out, int64_t out_stride, const void* in, int64_t in_stride, int64_t rows, int ff, int act_dtype,
+              void* stream);
 
 /* Rotary embedding on the first rot_dims coordinates of every head: pair i is the neighbours (2i, 2i + 1), or with
  * pair_halves != 0 the coordinates (i, i + rot_dims / 2); angle
@@ -214,11 +216,11 @@ int swm_capped_attention(void* out, const float* q, const void* key_cache, const
  * g * vdim: value_cache may point into the key cache (values that are a part of the key row).  Key and value sizes up
  * to 512.  Steps of few rows per sequence and few sequences share a tile's keys out among several workgroups, joined
  * by a second launch: `workspace` then holds swm_masked_attention_workspace_floats() floats (0: not such a step;
- * NULL: never shared out). */
+ * NULL: never shared out).  Output rows are out_stride >= heads * vdim elements apart. */
 int64_t swm_masked_attention_workspace_floats(int64_t rows, int num_seqs, int max_query_len, int heads, int kv_heads,
                                               int vdim, int page_size, int table_width, int window, int chunk);
-int swm_masked_attention(void* out, const float* q, const void* key_cache, const void* value_cache, const void* gate,
-                         int64_t gate_stride, const int32_t* block_tables, int table_width, const int32_t* q_start,
+int swm_masked_attention(void* out, int64_t out_stride, const float* q, const void* key_cache,
+                         const void* value_cache, const void* gate, int64_t gate_stride, const int32_t* block_tables, int table_width, const int32_t* q_start,
                          const int32_t* ctx_len, int64_t rows, int num_seqs, int max_query_len, int heads,
                          int kv_heads, int dim, int vdim, int page_size, float scale, float softcap, int window,
                          int chunk, int sink, int64_t k_stride, int64_t v_stride, float* workspace, int act_dtype,
@@ -342,12 +344,59 @@ int swm_sigmoid_attention(void* out, const float* q, const void* key_cache, cons
                           int max_query_len, int heads, int kv_heads, int dim, int vdim, int page_size, float scale,
                           int window, float* workspace, int act_dtype, void* stream);
 
-/* swm_group_router with the scores, the groups' scores and the weights named: softmax != 0: s = softmax(logits) over
- * all experts (else sigmoid); group_best_one != 0: a group scores its largest choice score (else the sum of its two
- * largest); normalize == 0: weights = s of the chosen * scale, not divided by their sum. */
+/* swm_group_router with the scores, the groups' scores and the weights named: softmax == SWM_ROUTER_SOFTMAX: s =
+ * softmax(logits) over all experts; SWM_ROUTER_SOFTMAX_CHOSEN: the choice goes by the logits themselves (+ correction) and
+ * s = exp(logit - largest logit), so that normalised weights are the softmax over the chosen logits; else sigmoid.
+ * group_best_one != 0: a group scores its largest choice score (else the sum of its two largest); normalize == 0: weights
+ * = s of the chosen * scale, not divided by their sum.  clear (NULL: nothing) fp32 [rows, clear_width] is set to zero: the
+ * rows that swm_expert_down_weighted adds into. */
+#define SWM_ROUTER_SOFTMAX 1
+#define SWM_ROUTER_SOFTMAX_CHOSEN 2
 int swm_group_router_as(int32_t* chosen, float* weights, const float* logits, const float* correction, int64_t rows,
                         int experts, int top, int groups, int keep, float scale, int softmax, int group_best_one,
-                        int normalize, void* stream);
+                        int normalize, float* clear, int clear_width, void* stream);
+
+/* ---- decoders that run a block of layers several times; latent attention with a query latent ---- */
+
+/* stream_out[t] (fp32) = scale * table[ids[t]] (table act_dtype [vocab, width]; an id beyond it gives NaN);
+ * rows_out (NULL: none) = the table's row, act_dtype; with `out`: out[t] = act_dtype(stream_out[t] /
+ * sqrt(mean(stream_out[t]^2) + eps) * (offset + weight)), weight fp32 [width]. */
+int swm_embed_stream(float* stream_out, void* rows_out, const int64_t* ids, const void* table, int64_t vocab, float scale,
+                     const float* weight, float offset, float eps, void* out, int64_t rows, int width, int act_dtype,
+                     void* stream);
+
+/* stream_io[t] += a[t] + b[t] + c[t] (as swm_stream_add_norm, a and b bf16); split[t] (bf16 [rows, 2 * width]) =
+ * bf16(v) | bf16(v - bf16(v)) of the new value v: the stream as a pair of bf16 numbers. */
+int swm_stream_split(float* stream_io, const void* a, int64_t a_stride, const void* b, int64_t b_stride, const float* c,
+                     void* split, int64_t rows, int width, void* stream);
+
+/* RMS norm per query and key head and the cache write of an attention layer without rotation: q_out (fp32 [rows, heads *
+ * dim]) = q / sqrt(mean(q^2) + eps) * q_weight per head, key_cache[slot] = the same of k with k_weight, value_cache[slot] = v
+ * (slot = slot_mapping[t], < 0: not cached).  Weights fp32 [dim] shared by the heads, NULL: none.  q, k, v are column
+ * ranges of one projection output (row stride in_stride).  Key and value sizes up to 512. */
+int swm_head_norm_cache(float* q_out, const void* q, const void* k, const void* v, int64_t in_stride, const float* q_weight,
+                        const float* k_weight, float eps, void* key_cache, void* value_cache, const int64_t* slot_mapping,
+                        int64_t rows, int heads, int kv_heads, int dim, int vdim, int act_dtype, void* stream);
+
+/* The two latents of a latent-attention layer, column ranges of one projection output (row stride in_stride):
+ * q_out[t] (act_dtype [rows, q_rank]) = q_down / sqrt(mean(.^2) + eps) * q_weight (q_rank 0: no query latent);
+ * cache[slot] (act_dtype [slots, rank + rot]) = kv_down[:rank] / sqrt(mean(.^2) + eps) * kv_weight | turned kv_down[rank:].
+ * Rotation: pair i is (i, i + rot / 2) when pair_halves != 0, else (2i, 2i + 1); it turns by float(position) * inv_freq[i]
+ * and is multiplied by amplitude. */
+int swm_latent_down(void* q_out, const void* q_down, int q_rank, const float* q_weight, const void* kv_down, int rank,
+                    const float* kv_weight, int64_t in_stride, float eps, const int64_t* positions,
+                    const float* inv_freq, int rot, int pair_halves, float amplitude, void* cache,
+                    const int64_t* slot_mapping, int64_t rows, int act_dtype, void* stream);
+
+/* A product per head with its neighbours fused: out[t, h, n] = sum_k b[h, n, k] a[t, h, k] for n < N (fp32 sums), then
+ * * sigmoid(gate) when gate != NULL (gate[t, h] when gate_per_head != 0, else gate[t, h * N + n]); out[t, h, N ..
+ * N + rot - 1] = q_rot[t, h] turned as in swm_latent_down (rot 0: none).  a, q_rot, out are addressed by row and head
+ * strides, gate by its row stride; b is contiguous [heads, N, K]; out_dtype is act_dtype or SW_F32. */
+int swm_head_project(void* out, int out_dtype, int64_t out_row, int64_t out_head, const void* a, int64_t a_row,
+                     int64_t a_head, const void* b, int N, int K, const void* q_rot, int64_t rot_row, int64_t rot_head,
+                     const int64_t* positions, const float* inv_freq, int rot, int pair_halves, float amplitude,
+                     const void* gate, int64_t gate_row, int gate_per_head, int64_t rows, int heads, int act_dtype,
+                     void* stream);
 
 #ifdef __cplusplus
 }

@@ -114,7 +114,7 @@ constexpr int max_waves_of(int nb) { return nb <= 4 ? 8 : 4; }
 
 template <typename T, int NB>
 __global__ __launch_bounds__(64 * max_waves_of(NB)) void capped_attention_kernel(
-    void* __restrict__ out, const float* __restrict__ q, const void* __restrict__ key_cache,
+    void* __restrict__ out, int64_t out_stride, const float* __restrict__ q, const void* __restrict__ key_cache,
     const void* __restrict__ value_cache, const void* __restrict__ gate, int64_t gate_stride,
     const int32_t* __restrict__ block_tables, int table_width, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_len, int num_seqs, int heads, int kv_heads, int dim, int vdim, int page_size,
@@ -350,7 +350,7 @@ __global__ __launch_bounds__(64 * max_waves_of(NB)) void capped_attention_kernel
       float v = sig ? num : num / den;
       const int64_t col = (int64_t)(g * R + hh) * vdim + c;
       if (gate != nullptr) v *= sigmoidf_(ld<T>(gate, (row0 + tt) * gate_stride + col));
-      st<T>(out, (row0 + tt) * (int64_t)heads * vdim + col, v);
+      st<T>(out, (row0 + tt) * out_stride + col, v);
     }
     return;
   }
@@ -374,7 +374,7 @@ __global__ __launch_bounds__(64 * max_waves_of(NB)) void capped_attention_kernel
     float v = Os[r * ostride + c];
     const int64_t col = (int64_t)(g * R + hh) * vdim + c;
     if (gate != nullptr) v *= sigmoidf_(ld<T>(gate, (row0 + tt) * gate_stride + col));
-    st<T>(out, (row0 + tt) * (int64_t)heads * vdim + col, v);
+    st<T>(out, (row0 + tt) * out_stride + col, v);
   }
 }
 
@@ -385,7 +385,7 @@ __global__ __launch_bounds__(64 * max_waves_of(NB)) void capped_attention_kernel
 // waves through LDS, both in a fixed order.  RQ: query rows (padded), C: coordinates per lane, U: keys in flight.
 template <typename T, int RQ, int C, int LK, int U>
 __global__ __launch_bounds__(512) void capped_attention_rows_kernel(
-    void* __restrict__ out, const float* __restrict__ q, const void* __restrict__ key_cache,
+    void* __restrict__ out, int64_t out_stride, const float* __restrict__ q, const void* __restrict__ key_cache,
     const void* __restrict__ value_cache, const void* __restrict__ gate, int64_t gate_stride,
     const int32_t* __restrict__ block_tables, int table_width, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_len, int heads, int kv_heads, int dim, int vdim, int page_size, int page_shift,
@@ -512,12 +512,12 @@ __global__ __launch_bounds__(512) void capped_attention_rows_kernel(
     float v = sig ? num : num / den;
     const int64_t col = (int64_t)(g * R + hh) * vdim + c;
     if (gate != nullptr) v *= sigmoidf_(ld<T>(gate, (row0 + tt) * gate_stride + col));
-    st<T>(out, (int64_t)(row0 + tt) * heads * vdim + col, v);
+    st<T>(out, (int64_t)(row0 + tt) * out_stride + col, v);
   }
 }
 
 template <typename T, int RQ, int C, int LK>
-int launch_capped_rows(void* out, const float* q, const void* key_cache, const void* value_cache, const void* gate,
+int launch_capped_rows(void* out, int64_t out_stride, const float* q, const void* key_cache, const void* value_cache, const void* gate,
                        int64_t gate_stride, const int32_t* block_tables, int table_width, const int32_t* q_start,
                        const int32_t* ctx_len, int num_seqs, int heads, int kv_heads, int dim, int vdim, int page_size,
                        float scale, float softcap, int window, int chunk, int sink, const float* score_bias, int64_t k_stride,
@@ -536,7 +536,7 @@ int launch_capped_rows(void* out, const float* q, const void* key_cache, const v
                                      (int)lds_bytes));
     raised = true;
   }
-  hipLaunchKernelGGL(kernel, dim3((unsigned)num_seqs, (unsigned)kv_heads), dim3(64 * nw), lds_bytes, stream, out, q,
+  hipLaunchKernelGGL(kernel, dim3((unsigned)num_seqs, (unsigned)kv_heads), dim3(64 * nw), lds_bytes, stream, out, out_stride, q,
                      key_cache, value_cache, gate, gate_stride, block_tables, table_width, q_start, ctx_len, heads,
                      kv_heads, dim, vdim, page_size, page_shift, scale, softcap, window, chunk, sink, score_bias, k_stride,
                      v_stride);
@@ -546,7 +546,7 @@ int launch_capped_rows(void* out, const float* q, const void* key_cache, const v
 
 // -> true when the step was taken by the vector-unit kernel (few rows, lanes' shares small enough for registers)
 template <typename T>
-bool try_capped_rows(int* status, int rows_used, void* out, const float* q, const void* key_cache,
+bool try_capped_rows(int* status, int rows_used, void* out, int64_t out_stride, const float* q, const void* key_cache,
                      const void* value_cache, const void* gate, int64_t gate_stride, const int32_t* block_tables,
                      int table_width, const int32_t* q_start, const int32_t* ctx_len, int num_seqs, int heads,
                      int kv_heads, int dim, int vdim, int page_size, float scale, float softcap, int window, int chunk,
@@ -564,7 +564,7 @@ bool try_capped_rows(int* status, int rows_used, void* out, const float* q, cons
   if (rq * c > 64) return false;
 #define SWM_ROWS_CASE(RQV, CV, LKV)                                                                                     \
   if (rq == RQV && c == CV && lk == LKV) {                                                                              \
-    *status = launch_capped_rows<T, RQV, CV, LKV>(out, q, key_cache, value_cache, gate, gate_stride, block_tables,      \
+    *status = launch_capped_rows<T, RQV, CV, LKV>(out, out_stride, q, key_cache, value_cache, gate, gate_stride, block_tables,      \
                                                   table_width, q_start, ctx_len, num_seqs, heads, kv_heads, dim, vdim,  \
                                                   page_size, scale, softcap, window, chunk, sink, score_bias, k_stride, \
                                                   v_stride, stream);                                                              \
@@ -583,7 +583,7 @@ bool try_capped_rows(int* status, int rows_used, void* out, const float* q, cons
 // (row, head), parts in a fixed order.
 template <typename T>
 __global__ __launch_bounds__(256) void capped_attention_join_kernel(
-    void* __restrict__ out, const float* __restrict__ partial, const void* __restrict__ gate, int64_t gate_stride,
+    void* __restrict__ out, int64_t out_stride, const float* __restrict__ partial, const void* __restrict__ gate, int64_t gate_stride,
     int64_t total_rows, int heads, int vdim, int parts, int sink, int sig) {
   const int64_t rh = blockIdx.x;                             // row * heads + head
   const float* ml = partial;
@@ -606,7 +606,7 @@ __global__ __launch_bounds__(256) void capped_attention_join_kernel(
     }
     float v = sig ? num : num / den;
     if (gate != nullptr) v *= sigmoidf_(ld<T>(gate, t * gate_stride + (int64_t)hd * vdim + c));
-    st<T>(out, rh * vdim + c, v);
+    st<T>(out, t * out_stride + (int64_t)hd * vdim + c, v);
   }
 }
 
@@ -627,7 +627,7 @@ inline int key_parts(int num_seqs, int max_query_len, int heads, int kv_heads, i
 }
 
 template <typename T, int NB>
-int launch_capped_attention(void* out, const float* q, const void* key_cache, const void* value_cache, const void* gate,
+int launch_capped_attention(void* out, int64_t out_stride, const float* q, const void* key_cache, const void* value_cache, const void* gate,
                             int64_t gate_stride, const int32_t* block_tables, int table_width, const int32_t* q_start,
                             const int32_t* ctx_len, int64_t rows, int num_seqs, int max_query_len, int heads,
                             int kv_heads, int dim, int vdim, int page_size, float scale, float softcap, int window,
@@ -640,7 +640,7 @@ int launch_capped_attention(void* out, const float* q, const void* key_cache, co
   const int rows_used = split ? max_query_len * R : kQT;
   if (split) {
     int status = SW_OK;
-    if (try_capped_rows<T>(&status, rows_used, out, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width,
+    if (try_capped_rows<T>(&status, rows_used, out, out_stride, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width,
                            q_start, ctx_len, num_seqs, heads, kv_heads, dim, vdim, page_size, scale, softcap, window,
                            chunk, sink, score_bias, k_stride, v_stride, stream))
       return status;
@@ -671,14 +671,14 @@ int launch_capped_attention(void* out, const float* q, const void* key_cache, co
   }
   const int64_t tiles = split ? num_seqs : (rows + tpt - 1) / tpt + num_seqs;
   const dim3 grid((unsigned)(split ? tiles : (tiles + nw - 1) / nw), (unsigned)kv_heads, (unsigned)parts);
-  hipLaunchKernelGGL(kernel, grid, dim3(64 * nw), lds_bytes(nw), stream, out, q, key_cache, value_cache, gate,
+  hipLaunchKernelGGL(kernel, grid, dim3(64 * nw), lds_bytes(nw), stream, out, out_stride, q, key_cache, value_cache, gate,
                      gate_stride, block_tables, table_width, q_start, ctx_len, num_seqs, heads, kv_heads, dim, vdim,
                      page_size, scale, softcap, window, chunk, sink, score_bias, k_stride, v_stride, tpt, split ? 1 : 0,
                      rows_used, page_shift, parts > 1 ? workspace : (float*)nullptr, rows);
   SW_CHECK_LAUNCH();
   if (parts > 1) {
     hipLaunchKernelGGL(capped_attention_join_kernel<T>, dim3((unsigned)(rows * heads)), dim3(vdim <= 64 ? 64 : 128), 0,
-                       stream, out, workspace, gate, gate_stride, rows, heads, vdim, parts, sink, score_bias != nullptr ? 1 : 0);
+                       stream, out, out_stride, workspace, gate, gate_stride, rows, heads, vdim, parts, sink, score_bias != nullptr ? 1 : 0);
     SW_CHECK_LAUNCH();
   }
   return SW_OK;
@@ -694,7 +694,7 @@ extern "C" int64_t swm_masked_attention_workspace_floats(int64_t rows, int num_s
   return parts > 1 ? (int64_t)parts * rows * heads * (vdim + 2) : 0;
 }
 
-static int masked_attention_impl(void* out, const float* q, const void* key_cache, const void* value_cache,
+static int masked_attention_impl(void* out, int64_t out_stride, const float* q, const void* key_cache, const void* value_cache,
                                  const void* gate, int64_t gate_stride, const int32_t* block_tables, int table_width,
                                  const int32_t* q_start, const int32_t* ctx_len, int64_t rows, int num_seqs,
                                  int max_query_len, int heads, int kv_heads, int dim, int vdim, int page_size,
@@ -714,12 +714,14 @@ static int masked_attention_impl(void* out, const float* q, const void* key_cach
   SW_CHECK_ARG(k_stride >= (int64_t)kv_heads * dim && v_stride >= (int64_t)kv_heads * vdim,
                "masked_attention: a cache slot of %lld / %lld elements cannot hold %d heads", (long long)k_stride,
                (long long)v_stride, kv_heads);
+  SW_CHECK_ARG(out_stride >= (int64_t)heads * vdim, "masked_attention: an output row of %lld elements cannot hold %d heads",
+               (long long)out_stride, heads);
   const int nvb = std::max((vdim + 31) / 32, (dim + 31) / 32);
   hipStream_t s = static_cast<hipStream_t>(stream);
 #define SWM_CAPPED_CASE(N)                                                                                              \
   case N:                                                                                                               \
     SWM_DISPATCH_ACT(act_dtype, return (launch_capped_attention<T, N>(                                                  \
-                                    out, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width,       \
+                                    out, out_stride, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width, \
                                     q_start, ctx_len, rows, num_seqs, max_query_len, heads, kv_heads, dim, vdim,        \
                                     page_size, scale, softcap, window, chunk, sink, score_bias, k_stride, v_stride,     \
                                     workspace, s)););                                                                              \
@@ -746,14 +748,14 @@ static int masked_attention_impl(void* out, const float* q, const void* key_cach
   return SW_OK;
 }
 
-extern "C" int swm_masked_attention(void* out, const float* q, const void* key_cache, const void* value_cache,
+extern "C" int swm_masked_attention(void* out, int64_t out_stride, const float* q, const void* key_cache, const void* value_cache,
                                     const void* gate, int64_t gate_stride, const int32_t* block_tables,
                                     int table_width, const int32_t* q_start, const int32_t* ctx_len, int64_t rows,
                                     int num_seqs, int max_query_len, int heads, int kv_heads, int dim, int vdim,
                                     int page_size, float scale, float softcap, int window, int chunk, int sink,
                                     int64_t k_stride, int64_t v_stride, float* workspace, int act_dtype, void* stream) {
-  return masked_attention_impl(out, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width, q_start,
-                               ctx_len, rows, num_seqs, max_query_len, heads, kv_heads, dim, vdim, page_size, scale,
+  return masked_attention_impl(out, out_stride, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width,
+                               q_start, ctx_len, rows, num_seqs, max_query_len, heads, kv_heads, dim, vdim, page_size, scale,
                                softcap, window, chunk, sink, nullptr, k_stride, v_stride, workspace, act_dtype, stream);
 }
 
@@ -767,7 +769,7 @@ extern "C" int swm_sigmoid_attention(void* out, const float* q, const void* key_
     sw::set_error("sigmoid_attention: the per-head bias is missing (a layer without one passes zeros)");
     return SW_ERR_INVALID;
   }
-  return masked_attention_impl(out, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width, q_start,
+  return masked_attention_impl(out, (int64_t)heads * vdim, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width, q_start,
                                ctx_len, rows, num_seqs, max_query_len, heads, kv_heads, dim, vdim, page_size, scale,
                                0.0f, window, 0, 0, score_bias, (int64_t)kv_heads * dim, (int64_t)kv_heads * vdim,
                                workspace, act_dtype, stream);
@@ -778,7 +780,7 @@ extern "C" int swm_capped_attention(void* out, const float* q, const void* key_c
                                     int table_width, const int32_t* q_start, const int32_t* ctx_len, int64_t rows,
                                     int num_seqs, int max_query_len, int heads, int kv_heads, int dim, int vdim, int page_size,
                                     float scale, float softcap, int window, int act_dtype, void* stream) {
-  return swm_masked_attention(out, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width, q_start,
+  return swm_masked_attention(out, (int64_t)heads * vdim, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width, q_start,
                               ctx_len, rows, num_seqs, max_query_len, heads, kv_heads, dim, vdim, page_size, scale,
                               softcap, window, 0, 0, (int64_t)kv_heads * dim, (int64_t)kv_heads * vdim, nullptr, act_dtype,
                               stream);

@@ -6,11 +6,11 @@
 // The host does not know how many rows an expert got (the sort stays on the device), so the grid has the
 // upper bound ceil(pairs / TM) + experts row tiles and each workgroup finds its (expert, tile) from the
 // prefix sums; surplus workgroups leave at once.  Tiles never straddle two experts.
-#include "mixers_common.cuh"
+#include "tile_gemm.cuh"
 
 namespace swm {
 
-constexpr int TM = 32, TN = 64, TK = 32, kFfnThreads = 256;
+constexpr int kFfnThreads = kTileThreads;
 
 __device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
 // activation of an expert's hidden layer: SWM_ACT_GELU (exact gelu), SWM_ACT_RELU2 (the square of relu) or
@@ -52,48 +52,6 @@ __device__ __forceinline__ int find_tile(const int32_t* __restrict__ expert_star
   return 0;
 }
 
-// acc[2][4] of thread (ty, tx): rows 2 * ty + {0, 1}, columns tx + 16 * {0..3} of the tile
-//   A row p: a_base + a_row(p) * K        B row n: b_base + n * K
-template <typename T, typename RowOf>
-__device__ __forceinline__ void tile_gemm(float (&acc)[2][4], const void* __restrict__ a, RowOf a_row, int rows,
-                                          const void* __restrict__ b, int64_t b_off, int n0, int N, int K,
-                                          float (*As)[TK + 1], float (*Bs)[TK + 1]) {
-  const int tid = threadIdx.x, ty = tid >> 4, tx = tid & 15;
-#pragma unroll
-  for (int i = 0; i < 2; ++i)
-#pragma unroll
-    for (int j = 0; j < 4; ++j) acc[i][j] = 0.0f;
-  for (int k0 = 0; k0 < K; k0 += TK) {
-    // A tile: 32 x 32 = 1024 values, 4 per thread; B tile: 64 x 32 = 2048 values, 8 per thread
-#pragma unroll
-    for (int it = 0; it < 4; ++it) {
-      const int e = tid + it * kFfnThreads, r = e >> 5, k = e & 31;
-      float v = 0.0f;
-      if (r < rows && k0 + k < K) v = ld<T>(a, a_row(r) * (int64_t)K + k0 + k);
-      As[r][k] = v;
-    }
-#pragma unroll
-    for (int it = 0; it < 8; ++it) {
-      const int e = tid + it * kFfnThreads, r = e >> 5, k = e & 31;
-      float v = 0.0f;
-      if (n0 + r < N && k0 + k < K) v = ld<T>(b, b_off + (int64_t)(n0 + r) * K + k0 + k);
-      Bs[r][k] = v;
-    }
-    __syncthreads();
-#pragma unroll
-    for (int k = 0; k < TK; ++k) {
-      const float a0 = As[2 * ty][k], a1 = As[2 * ty + 1][k];
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const float bv = Bs[tx + 16 * j][k];
-        acc[0][j] += a0 * bv;
-        acc[1][j] += a1 * bv;
-      }
-    }
-    __syncthreads();
-  }
-}
-
 template <typename T>
 __global__ __launch_bounds__(kFfnThreads) void expert_up_gelu_kernel(
     void* __restrict__ hidden, const void* __restrict__ x, const void* __restrict__ up,
@@ -106,7 +64,7 @@ __global__ __launch_bounds__(kFfnThreads) void expert_up_gelu_kernel(
   if (rows == 0) return;
   const int n0 = blockIdx.y * TN;
   float acc[2][4];
-  tile_gemm<T>(acc, x, [&](int r) { return (int64_t)(order[row0 + r] / top); }, rows, up, (int64_t)e * up_rows * width, n0,
+  tile_gemm<T>(acc, x, [&](int r) { return (int64_t)(order[row0 + r] / top) * width; }, rows, up, (int64_t)e * up_rows * width, n0,
                up_rows, width, As, Bs);
   const int ty = threadIdx.x >> 4, tx = threadIdx.x & 15;
 #pragma unroll
@@ -142,7 +100,7 @@ __global__ __launch_bounds__(kFfnThreads) void expert_down_kernel(
   if (rows == 0) return;
   const int n0 = blockIdx.y * TN;
   float acc[2][4];
-  tile_gemm<T>(acc, hidden, [&](int r) { return (int64_t)(row0 + r); }, rows, down, (int64_t)e * width * ff, n0, width,
+  tile_gemm<T>(acc, hidden, [&](int r) { return (int64_t)(row0 + r) * ff; }, rows, down, (int64_t)e * width * ff, n0, width,
                ff, As, Bs);
   const int ty = threadIdx.x >> 4, tx = threadIdx.x & 15;
 #pragma unroll
@@ -165,53 +123,6 @@ __global__ __launch_bounds__(kFfnThreads) void expert_down_kernel(
 
 
 // ------------------------------------------------------------------------------- bf16 on the matrix cores
-// 64 x 64 output tile per workgroup, one 32 x 32 quadrant per wave (v_mfma_f32_32x32x16_bf16, fp32 accumulation);
-// stages of 64 reduction steps go global -> LDS as 16-byte vectors.  Both operands are contiguous along the
-// reduction and are read with the SAME lane -> k mapping (8 consecutive k per lane, the wave's halves 8 apart),
-// so only the accumulator's layout matters: element i of lane l is row 8 * (i / 4) + 4 * (l / 32) + i % 4,
-// column l % 32.  Needs the reduction size to be a multiple of 8.
-constexpr int MM = 64, MN = 64, MK = 64, MPAD = 8;
-using bf16x8 = __attribute__((ext_vector_type(8))) __bf16;
-using f32x16 = __attribute__((ext_vector_type(16))) float;
-
-template <typename RowOf>
-__device__ __forceinline__ void tile_gemm_mfma(f32x16& acc, const uint16_t* __restrict__ a, RowOf a_row, int rows,
-                                               const uint16_t* __restrict__ b, int64_t b_off, int n0, int N, int K,
-                                               uint16_t (*As)[MK + MPAD], uint16_t (*Bs)[MK + MPAD]) {
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
-  const int wm = wave >> 1, wn = wave & 1;
-#pragma unroll
-  for (int i = 0; i < 16; ++i) acc[i] = 0.0f;
-  for (int k0 = 0; k0 < K; k0 += MK) {
-#pragma unroll
-    for (int it = 0; it < 2; ++it) {
-      const int e = tid + it * kFfnThreads, r = e >> 3, k = (e & 7) * 8;
-      uint4 va = make_uint4(0u, 0u, 0u, 0u), vb = make_uint4(0u, 0u, 0u, 0u);
-      if (r < rows && k0 + k < K) va = *reinterpret_cast<const uint4*>(a + a_row(r) * (int64_t)K + k0 + k);
-      if (n0 + r < N && k0 + k < K) vb = *reinterpret_cast<const uint4*>(b + b_off + (int64_t)(n0 + r) * K + k0 + k);
-      *reinterpret_cast<uint4*>(&As[r][k]) = va;
-      *reinterpret_cast<uint4*>(&Bs[r][k]) = vb;
-    }
-    __syncthreads();
-#pragma unroll
-    for (int ks = 0; ks < MK; ks += 16) {
-      const bf16x8 av = *reinterpret_cast<const bf16x8*>(&As[wm * 32 + (lane & 31)][ks + 8 * (lane >> 5)]);
-      const bf16x8 bv = *reinterpret_cast<const bf16x8*>(&Bs[wn * 32 + (lane & 31)][ks + 8 * (lane >> 5)]);
-      acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(av, bv, acc, 0, 0, 0);
-    }
-    __syncthreads();
-  }
-}
-
-// calls f(row in tile, column in tile, value) for the 16 accumulator elements of this lane
-template <typename F>
-__device__ __forceinline__ void for_each_acc(const f32x16& acc, F&& f) {
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const int wm = wave >> 1, wn = wave & 1;
-#pragma unroll
-  for (int i = 0; i < 16; ++i) f(wm * 32 + 8 * (i / 4) + 4 * (lane >> 5) + (i % 4), wn * 32 + (lane & 31), acc[i]);
-}
-
 __global__ __launch_bounds__(kFfnThreads) void expert_up_gelu_mfma_kernel(
     uint16_t* __restrict__ hidden, const uint16_t* __restrict__ x, const uint16_t* __restrict__ up,
     const int32_t* __restrict__ order, const int32_t* __restrict__ expert_start, int num_experts, int width, int ff,
@@ -223,7 +134,7 @@ __global__ __launch_bounds__(kFfnThreads) void expert_up_gelu_mfma_kernel(
   if (rows == 0) return;
   const int n0 = blockIdx.y * MN;
   f32x16 acc;
-  tile_gemm_mfma(acc, x, [&](int r) { return (int64_t)(order[row0 + r] / top); }, rows, up, (int64_t)e * up_rows * width,
+  tile_gemm_mfma<true>(acc, x, [&](int r) { return (int64_t)(order[row0 + r] / top) * width; }, rows, up, (int64_t)e * up_rows * width,
                  n0, up_rows, width, As, Bs);
   if (activation == SWM_ACT_CLAMPED_GLU) {
     // a lane's column c of the tile: c % 32 < 16 is the gate product of channel (n0 + c) / 32 * 16 + c % 16, and lane
@@ -252,7 +163,7 @@ __global__ __launch_bounds__(kFfnThreads) void expert_down_mfma_kernel(
   if (rows == 0) return;
   const int n0 = blockIdx.y * MN;
   f32x16 acc;
-  tile_gemm_mfma(acc, hidden, [&](int r) { return (int64_t)(row0 + r); }, rows, down, (int64_t)e * width * ff, n0, width,
+  tile_gemm_mfma<true>(acc, hidden, [&](int r) { return (int64_t)(row0 + r) * ff; }, rows, down, (int64_t)e * width * ff, n0, width,
                  ff, As, Bs);
   for_each_acc(acc, [&](int r, int c, float v) {
     if (r < rows && n0 + c < width) {

@@ -4,6 +4,7 @@
 //   * clamped_glu / relu2: activations between the library GEMMs of a feed-forward;
 //   * rope_cache: partial rotary embedding on neighbouring pairs from a table of per-pair frequencies (angles
 //     from fp32 positions), rotated queries out in fp32, rotated keys and values into the paged cache;
+//   * head_norm_cache: queries and keys normed per head, unrotated, out in fp32 / into the paged cache;
 //   * group_router: the choice of a sigmoid router from its fp32 logits: a selection bias, a limit to the best
 //     groups of experts and weights normalised over the chosen ones.
 // All arithmetic is fp32; activations are read and written in the model's dtype.
@@ -57,12 +58,31 @@ __global__ __launch_bounds__(kPbThreads) void clamped_glu_kernel(void* __restric
 }
 
 template <typename T>
-__global__ __launch_bounds__(kPbThreads) void relu2_kernel(void* __restrict__ out, const void* __restrict__ in,
-                                                           int64_t in_stride, int ff) {
+__global__ __launch_bounds__(kPbThreads) void relu2_kernel(void* __restrict__ out, int64_t out_stride,
+                                                           const void* __restrict__ in, int64_t in_stride, int ff) {
   const int64_t t = blockIdx.x;
   for (int i = blockIdx.y * kPbThreads + threadIdx.x; i < ff; i += gridDim.y * kPbThreads) {
     const float z = fmaxf(ld<T>(in, t * in_stride + i), 0.0f);
-    st<T>(out, t * (int64_t)ff + i, z * z);
+    st<T>(out, t * out_stride + i, z * z);
+  }
+}
+
+// the same over runs of 16 bytes: rows that begin and end at multiples of 16 bytes
+template <typename T>
+__global__ __launch_bounds__(kPbThreads) void relu2_vec_kernel(void* __restrict__ out, int64_t out_stride,
+                                                               const void* __restrict__ in, int64_t in_stride, int ff) {
+  using S = typename Conv<T>::store_t;
+  constexpr int V = 16 / sizeof(S);
+  const int64_t t = blockIdx.x;
+  for (int i = blockIdx.y * kPbThreads + threadIdx.x; i < ff / V; i += gridDim.y * kPbThreads) {
+    S x[V], y[V];
+    *reinterpret_cast<uint4*>(x) = *reinterpret_cast<const uint4*>(static_cast<const S*>(in) + t * in_stride + i * V);
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      const float z = fmaxf(Conv<T>::to_float(x[j]), 0.0f);
+      y[j] = Conv<T>::from_float(z * z);
+    }
+    *reinterpret_cast<uint4*>(static_cast<S*>(out) + t * out_stride + i * V) = *reinterpret_cast<const uint4*>(y);
   }
 }
 
@@ -184,6 +204,72 @@ __global__ __launch_bounds__(kPbThreads) void rope_cache_kernel(
     st<T>(value_cache, slot * (int64_t)kv_heads * vdim + e, ld<T>(v, row + e));
 }
 
+// Queries and keys that are normed per head and NOT rotated: a wave owns one (row, head) and keeps the head's coordinates
+// in registers, so every number is read once.  Units of a row: query heads, key heads, value heads (copied).  V: neighbours
+// per access (2: sizes, strides and bases are even).
+constexpr int kMaxHeadSize = 512;
+
+template <typename T, int V>
+__global__ __launch_bounds__(kPbThreads) void head_norm_cache_kernel(
+    float* __restrict__ q_out, const void* __restrict__ q, const void* __restrict__ k, const void* __restrict__ v,
+    int64_t in_stride, const float* __restrict__ q_weight, const float* __restrict__ k_weight, float eps,
+    void* __restrict__ key_cache, void* __restrict__ value_cache, const int64_t* __restrict__ slot_mapping, int heads,
+    int kv_heads, int dim, int vdim) {
+  using S = typename Conv<T>::store_t;
+  struct alignas(V * sizeof(S)) Piece { S x[V]; };
+  struct alignas(V * sizeof(float)) Piece32 { float x[V]; };
+  constexpr int PER = kMaxHeadSize / 64 / V;                 // pieces of a lane
+  const int64_t t = blockIdx.x;
+  const int lane = threadIdx.x & 63, unit = blockIdx.y * (kPbThreads / 64) + (threadIdx.x >> 6);
+  if (unit >= heads + 2 * kv_heads) return;                  // no barrier below
+  const bool is_q = unit < heads, is_v = unit >= heads + kv_heads;
+  const int hd = is_q ? unit : is_v ? unit - heads - kv_heads : unit - heads, size = is_v ? vdim : dim;
+  int64_t slot = 0;
+  if (!is_q && (slot = slot_mapping[t]) < 0) return;
+  const S* src = static_cast<const S*>(is_q ? q : is_v ? v : k) + t * in_stride + (int64_t)hd * size;
+  Piece r[PER];
+  float ss = 0.0f;
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int c = (lane + 64 * j) * V;
+    if (c < size) {
+      r[j] = *reinterpret_cast<const Piece*>(src + c);
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        const float x = Conv<T>::to_float(r[j].x[e]);
+        ss += x * x;
+      }
+    }
+  }
+  if (is_v) {
+    S* dst = static_cast<S*>(value_cache) + (slot * kv_heads + hd) * size;
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int c = (lane + 64 * j) * V;
+      if (c < size) *reinterpret_cast<Piece*>(dst + c) = r[j];
+    }
+    return;
+  }
+  const float f = 1.0f / sqrtf(sw::wave_sum(ss) / (float)size + eps);
+  const float* w = is_q ? q_weight : k_weight;
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int c = (lane + 64 * j) * V;
+    if (c >= size) continue;
+    Piece32 o;
+#pragma unroll
+    for (int e = 0; e < V; ++e) o.x[e] = Conv<T>::to_float(r[j].x[e]) * f * (w != nullptr ? w[c + e] : 1.0f);
+    if (is_q) {
+      *reinterpret_cast<Piece32*>(q_out + (t * heads + hd) * (int64_t)size + c) = o;
+    } else {
+      Piece p;
+#pragma unroll
+      for (int e = 0; e < V; ++e) p.x[e] = Conv<T>::from_float(o.x[e]);
+      *reinterpret_cast<Piece*>(static_cast<S*>(key_cache) + (slot * kv_heads + hd) * size + c) = p;
+    }
+  }
+}
+
 // The choice of one row by one wave: scores by the lanes, the choice by lane 0 (a few hundred LDS reads for the usual
 // sizes).  logits: the row's `experts` numbers (global or LDS); score, choice: LDS scratch of the wave.
 constexpr int kMaxRouterExperts = 256;
@@ -193,7 +279,8 @@ __device__ __forceinline__ void router_choice(int lane, const float* __restrict_
                                               int keep, float scale, int softmax, int group_best_one, int normalize,
                                               int32_t* __restrict__ chosen, float* __restrict__ weights) {
   float top_logit = 0.0f, inv_sum = 1.0f;
-  if (softmax) {                                             // scores: the softmax over ALL experts
+  const bool by_logit = softmax == SWM_ROUTER_SOFTMAX_CHOSEN;
+  if (softmax) {                                             // scores: the softmax over ALL experts (or its numerators)
     float m = -INFINITY;
     for (int e = lane; e < experts; e += 64) m = fmaxf(m, logits[e]);
     for (int off = 32; off > 0; off >>= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
@@ -204,9 +291,9 @@ __device__ __forceinline__ void router_choice(int lane, const float* __restrict_
   }
   for (int e = lane; e < experts; e += 64) {
     const float z = logits[e];
-    const float s = softmax ? expf(z - top_logit) * inv_sum : sigmoidf_(z);
+    const float s = softmax ? expf(z - top_logit) * (by_logit ? 1.0f : inv_sum) : sigmoidf_(z);
     score[e] = s;
-    choice[e] = s + (correction != nullptr ? correction[e] : 0.0f);
+    choice[e] = (by_logit ? z : s) + (correction != nullptr ? correction[e] : 0.0f);
   }
   __builtin_amdgcn_wave_barrier();
   __threadfence_block();
@@ -284,12 +371,14 @@ __device__ __forceinline__ void router_choice(int lane, const float* __restrict_
 __global__ __launch_bounds__(256) void group_router_kernel(
     int32_t* __restrict__ chosen, float* __restrict__ weights, const float* __restrict__ logits,
     const float* __restrict__ correction, int64_t rows, int experts, int top, int groups, int keep, float scale,
-    int softmax, int group_best_one, int normalize) {
+    int softmax, int group_best_one, int normalize, float* __restrict__ clear, int clear_width) {
   __shared__ float s_score[4][kMaxRouterExperts];
   __shared__ float s_choice[4][kMaxRouterExperts];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int64_t t = (int64_t)blockIdx.x * 4 + wave;
   if (t >= rows) return;                                     // uniform over the wave; no workgroup barrier below
+  if (clear != nullptr)
+    for (int i = lane; i < clear_width; i += 64) clear[t * clear_width + i] = 0.0f;
   router_choice(lane, logits + t * experts, s_score[wave], s_choice[wave], correction, experts, top, groups, keep, scale,
                 softmax, group_best_one, normalize, chosen + t * top, weights + t * top);
 }
@@ -355,14 +444,24 @@ int swm_clamped_glu(void* out, const void* in, int64_t in_stride, int64_t rows, 
   return SW_OK;
 }
 
-int swm_relu2(void* out, const void* in, int64_t in_stride, int64_t rows, int ff, int act_dtype, void* stream) {
+int swm_relu2(void* out, int64_t out_stride, const void* in, int64_t in_stride, int64_t rows, int ff, int act_dtype,
+              void* stream) {
   using namespace swm;
   if (rows == 0) return SW_OK;
   SW_CHECK_ARG(act_ok(act_dtype), "relu2: unsupported dtype %d", act_dtype);
-  SW_CHECK_ARG(ff > 0 && rows < (1ll << 31), "relu2: bad shape");
+  SW_CHECK_ARG(ff > 0 && out_stride >= ff && rows < (1ll << 31), "relu2: bad shape");
+  const int v = act_dtype == SW_F32 ? 4 : 8;
+  if (ff % v == 0 && in_stride % v == 0 && out_stride % v == 0 && reinterpret_cast<uintptr_t>(in) % 16 == 0 &&
+      reinterpret_cast<uintptr_t>(out) % 16 == 0) {
+    const dim3 grid((unsigned)rows, (unsigned)std::min(8, (ff / v + kPbThreads - 1) / kPbThreads));
+    SWM_DISPATCH_ACT(act_dtype, hipLaunchKernelGGL(relu2_vec_kernel<T>, grid, dim3(kPbThreads), 0,
+                                                   static_cast<hipStream_t>(stream), out, out_stride, in, in_stride, ff););
+    SW_CHECK_LAUNCH();
+    return SW_OK;
+  }
   const dim3 grid((unsigned)rows, (unsigned)std::min(8, (ff + kPbThreads - 1) / kPbThreads));
   SWM_DISPATCH_ACT(act_dtype, hipLaunchKernelGGL(relu2_kernel<T>, grid, dim3(kPbThreads), 0,
-                                                 static_cast<hipStream_t>(stream), out, in, in_stride, ff););
+                                                 static_cast<hipStream_t>(stream), out, out_stride, in, in_stride, ff););
   SW_CHECK_LAUNCH();
   return SW_OK;
 }
@@ -400,17 +499,51 @@ int swm_norm_rope_cache(float* q_out, const void* q, const void* k, const void* 
   return SW_OK;
 }
 
+int swm_head_norm_cache(float* q_out, const void* q, const void* k, const void* v, int64_t in_stride, const float* q_weight,
+                        const float* k_weight, float eps, void* key_cache, void* value_cache, const int64_t* slot_mapping,
+                        int64_t rows, int heads, int kv_heads, int dim, int vdim, int act_dtype, void* stream) {
+  using namespace swm;
+  if (rows == 0) return SW_OK;
+  SW_CHECK_ARG(act_ok(act_dtype), "head_norm_cache: unsupported dtype %d", act_dtype);
+  SW_CHECK_ARG(heads > 0 && kv_heads > 0 && dim > 0 && dim <= kMaxHeadSize && vdim > 0 && vdim <= kMaxHeadSize &&
+                   rows < (1ll << 31),
+               "head_norm_cache: %d and %d heads of key size %d, value size %d (at most %d each)", heads, kv_heads, dim, vdim,
+               kMaxHeadSize);
+  SW_CHECK_ARG(q != nullptr && k != nullptr && v != nullptr && q_out != nullptr && key_cache != nullptr &&
+                   value_cache != nullptr && slot_mapping != nullptr,
+               "head_norm_cache: a part is missing");
+  const uintptr_t piece = act_dtype == SW_F32 ? 8 : 4;
+  auto even = [&](const void* p) { return reinterpret_cast<uintptr_t>(p) % piece == 0; };
+  const bool pairs = dim % 2 == 0 && vdim % 2 == 0 && in_stride % 2 == 0 && even(q) && even(k) && even(v) &&
+                     even(key_cache) && even(value_cache);
+  const dim3 grid((unsigned)rows, (unsigned)((heads + 2 * kv_heads + kPbThreads / 64 - 1) / (kPbThreads / 64)));
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (pairs) {
+    SWM_DISPATCH_ACT(act_dtype, hipLaunchKernelGGL((head_norm_cache_kernel<T, 2>), grid, dim3(kPbThreads), 0, s, q_out, q, k,
+                                                   v, in_stride, q_weight, k_weight, eps, key_cache, value_cache,
+                                                   slot_mapping, heads, kv_heads, dim, vdim););
+  } else {
+    SWM_DISPATCH_ACT(act_dtype, hipLaunchKernelGGL((head_norm_cache_kernel<T, 1>), grid, dim3(kPbThreads), 0, s, q_out, q, k,
+                                                   v, in_stride, q_weight, k_weight, eps, key_cache, value_cache,
+                                                   slot_mapping, heads, kv_heads, dim, vdim););
+  }
+  SW_CHECK_LAUNCH();
+  return SW_OK;
+}
+
 int swm_group_router(int32_t* chosen, float* weights, const float* logits, const float* correction, int64_t rows,
                      int experts, int top, int groups, int keep, float scale, void* stream) {
   return swm_group_router_as(chosen, weights, logits, correction, rows, experts, top, groups, keep, scale, 0, 0, 1,
-                             stream);
+                             nullptr, 0, stream);
 }
 
 int swm_group_router_as(int32_t* chosen, float* weights, const float* logits, const float* correction, int64_t rows,
                         int experts, int top, int groups, int keep, float scale, int softmax, int group_best_one,
-                        int normalize, void* stream) {
+                        int normalize, float* clear, int clear_width, void* stream) {
   using namespace swm;
   if (rows == 0) return SW_OK;
+  SW_CHECK_ARG(softmax >= 0 && softmax <= SWM_ROUTER_SOFTMAX_CHOSEN && (clear == nullptr || clear_width > 0),
+               "group_router: unknown score %d, or a row of no width to clear", softmax);
   SW_CHECK_ARG(experts > 0 && experts <= kMaxRouterExperts && top > 0 && top <= experts,
                "group_router: %d experts (1..%d supported), top %d", experts, kMaxRouterExperts, top);
   SW_CHECK_ARG(groups >= 1 && keep >= 1 && keep <= groups && experts % groups == 0 &&
@@ -418,7 +551,7 @@ int swm_group_router_as(int32_t* chosen, float* weights, const float* logits, co
                "group_router: %d groups, %d kept, %d experts, top %d", groups, keep, experts, top);
   hipLaunchKernelGGL(group_router_kernel, dim3((unsigned)((rows + 3) / 4)), dim3(256), 0, static_cast<hipStream_t>(stream),
                      chosen, weights, logits, correction, rows, experts, top, groups, keep, scale, softmax, group_best_one,
-                     normalize);
+                     normalize, clear, clear_width);
   SW_CHECK_LAUNCH();
   return SW_OK;
 }

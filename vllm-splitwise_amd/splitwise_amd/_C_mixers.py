@@ -12,13 +12,13 @@ import ctypes
 import os
 import subprocess
 from types import SimpleNamespace
-from typing import Optional
+from typing import Optional, Union
 
 import torch
 
 _PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 _LIB_PATH = os.path.join(_PKG_DIR, "libsplitwise_mixers.so")
-ABI_VERSION = 5
+ABI_VERSION = 6
 
 SW_F32, SW_BF16 = 0, 2
 _ACT = {torch.float32: SW_F32, torch.bfloat16: SW_BF16}
@@ -41,13 +41,13 @@ _SIGNATURES = {
     "swm_expert_down_weighted": [_p, _p, _p, _p, _p, _i, _l, _i, _i, _i, _f, _p, _i, _p],
     "swm_stream_add_norm": [_p, _p, _l, _p, _l, _p, _p, _f, _f, _p, _l, _i, _i, _p],
     "swm_clamped_glu": [_p, _p, _l, _l, _i, _f, _f, _f, _i, _p],
-    "swm_relu2": [_p, _p, _l, _l, _i, _i, _p],
+    "swm_relu2": [_p, _l, _p, _l, _l, _i, _i, _p],
     "swm_rope_cache": [_p, _p, _p, _p, _l, _p, _p, _i, _i, _p, _p, _p, _l, _i, _i, _i, _i, _i, _p],
     "swm_group_router": [_p, _p, _p, _p, _l, _i, _i, _i, _i, _f, _p],
     "swm_group_pairs": [_p, _p, _p, _l, _i, _p],
     "swm_capped_attention": [_p, _p, _p, _p, _p, _l, _p, _i, _p, _p, _l, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i,
                              _p],
-    "swm_masked_attention": [_p, _p, _p, _p, _p, _l, _p, _i, _p, _p, _l, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i,
+    "swm_masked_attention": [_p, _l, _p, _p, _p, _p, _l, _p, _i, _p, _p, _l, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i,
                              _i, _l, _l, _p, _i, _p],
     "swm_gated_stream_step": [_p, _p, _l, _p, _l, _f, _p, _l, _p, _i, _p, _p, _p, _p, _l, _i, _i, _p],
     "swm_poly_norm": [_p, _p, _l, _p, _f, _l, _i, _i, _p],
@@ -63,10 +63,17 @@ _SIGNATURES = {
     "swm_norm_rope_cache": [_p, _p, _p, _p, _l, _p, _p, _f, _p, _p, _i, _i, _p, _p, _p, _l, _i, _i, _i, _i, _i, _p],
     "swm_sigmoid_attention": [_p, _p, _p, _p, _p, _l, _p, _p, _i, _p, _p, _l, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p,
                               _i, _p],
-    "swm_group_router_as": [_p, _p, _p, _p, _l, _i, _i, _i, _i, _f, _i, _i, _i, _p],
+    "swm_group_router_as": [_p, _p, _p, _p, _l, _i, _i, _i, _i, _f, _i, _i, _i, _p, _i, _p],
+    "swm_embed_stream": [_p, _p, _p, _p, _l, _f, _p, _f, _f, _p, _l, _i, _i, _p],
+    "swm_stream_split": [_p, _p, _l, _p, _l, _p, _p, _l, _i, _p],
+    "swm_head_norm_cache": [_p, _p, _p, _p, _l, _p, _p, _f, _p, _p, _p, _l, _i, _i, _i, _i, _i, _p],
+    "swm_latent_down": [_p, _p, _i, _p, _p, _i, _p, _l, _f, _p, _p, _i, _i, _f, _p, _p, _l, _i, _p],
+    "swm_head_project": [_p, _i, _l, _l, _p, _l, _l, _p, _i, _i, _p, _l, _l, _p, _p, _i, _i, _f, _p, _l, _i, _l, _i, _i,
+                         _p],
     "swm_expert_up_as": [_p, _p, _p, _p, _p, _i, _l, _i, _i, _i, _i, _f, _f, _f, _i, _p],
 }
 ACT_GELU, ACT_RELU2, ACT_NONE, ACT_CLAMPED_GLU = 0, 1, 2, 3
+ROUTER_SOFTMAX, ROUTER_SOFTMAX_CHOSEN = 1, 2
 
 _lib = None
 
@@ -554,11 +561,12 @@ def clamped_glu(out: torch.Tensor, gate_up: torch.Tensor, alpha: float, limit: f
 
 
 def relu2(out: torch.Tensor, x: torch.Tensor) -> None:
+    """out = max(x, 0)^2; both 2-D views (column ranges of wider rows are fine)."""
     _dev(out, x)
-    _need(out.is_contiguous() and x.shape == out.shape and x.dtype == out.dtype and out.dim() == 2, "relu2: shapes")
+    _need(x.shape == out.shape and x.dtype == out.dtype and out.dim() == 2, "relu2: shapes")
     with _on_device_of(out):
-        _check(load_library().swm_relu2(out.data_ptr(), x.data_ptr(), _rows(x, "x"), out.shape[0], out.shape[1],
-                                        _act(out), _stream(out)))
+        _check(load_library().swm_relu2(out.data_ptr(), _rows(out, "out"), x.data_ptr(), _rows(x, "x"), out.shape[0],
+                                        out.shape[1], _act(out), _stream(out)))
 
 
 def rope_cache(q_out: torch.Tensor, q: torch.Tensor, k: Optional[torch.Tensor], v: Optional[torch.Tensor],
@@ -612,12 +620,15 @@ def rope_cache(q_out: torch.Tensor, q: torch.Tensor, k: Optional[torch.Tensor], 
 
 
 def group_router(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int, keep: int,
-                 scale: float, softmax: bool = False, group_best_one: bool = False, normalize: bool = True):
+                 scale: float, softmax: Union[bool, int] = False, group_best_one: bool = False, normalize: bool = True,
+                 clear: Optional[torch.Tensor] = None):
     """logits fp32 [rows, experts] -> (chosen int32 [rows, top], weights fp32 [rows, top]).  Scores: sigmoid of the
     logits, or with ``softmax`` their softmax over all experts; a group scores the sum of its two best choice scores,
     or with ``group_best_one`` its best; the chosen experts' scores are divided by their sum unless ``normalize`` is
-    off; all times ``scale``."""
-    _dev(logits, correction)
+    off; all times ``scale``.  ``softmax`` = ROUTER_SOFTMAX_CHOSEN: the choice goes by the logits themselves and the
+    (normalised) weights are the softmax over the chosen ones.  ``clear`` (fp32 [rows, width]) is set to zero in the same
+    launch: the sum that ``expert_ffn`` adds into."""
+    _dev(logits, correction, clear)
     _f32c(logits, "logits")
     rows, experts = logits.shape
     if correction is not None:
@@ -625,11 +636,15 @@ def group_router(logits: torch.Tensor, correction: Optional[torch.Tensor], top: 
         _need(correction.numel() == experts, "group_router: correction")
     chosen = torch.empty(rows, top, dtype=torch.int32, device=logits.device)
     weights = torch.empty(rows, top, dtype=torch.float32, device=logits.device)
+    if clear is not None:
+        _f32c(clear, "clear")
+        _need(clear.dim() == 2 and clear.shape[0] == rows, "group_router: one row to clear per row of logits")
     with _on_device_of(logits):
         _check(load_library().swm_group_router_as(chosen.data_ptr(), weights.data_ptr(), logits.data_ptr(),
                                                   _opt_ptr(correction), rows, experts, top, groups, keep, scale,
-                                                  1 if softmax else 0, 1 if group_best_one else 0,
-                                                  1 if normalize else 0, _stream(logits)))
+                                                  int(softmax), 1 if group_best_one else 0, 1 if normalize else 0,
+                                                  _opt_ptr(clear), 0 if clear is None else clear.shape[1],
+                                                  _stream(logits)))
     return chosen, weights
 
 
@@ -651,8 +666,8 @@ def capped_attention(out: torch.Tensor, q: torch.Tensor, key_cache: torch.Tensor
                      gate: Optional[torch.Tensor], batch, heads: int, kv_heads: int, dim: int, vdim: int, scale: float,
                      softcap: float = 0.0, window: int = 0, chunk: int = 0, sink: bool = False,
                      score_bias: Optional[torch.Tensor] = None) -> None:
-    """out [rows, heads * vdim] (cache dtype); q fp32 [rows, heads * dim]; caches [pages, page, kv_heads * size];
-    gate (None: no gate): a 2-D view [rows, heads * vdim] in the cache dtype.  ``window`` / ``chunk``: the mask (a
+    """out [rows, heads * vdim] (cache dtype; a column range of wider rows is fine, but not with ``score_bias``); q fp32
+    [rows, heads * dim]; caches [pages, page, kv_heads * size]; gate (None: no gate): a 2-D view [rows, heads * vdim] in the cache dtype.  ``window`` / ``chunk``: the mask (a
     sliding window, or chunks counted from position 0; neither: plain causal); ``sink``: one more term exp(0) in the
     softmax's denominator.  ``value_cache`` None: a token's values are the first kv_heads * vdim elements of its
     key row (attention over a shared latent).  ``score_bias`` (fp32 [heads]): no softmax -- a seen key weighs
@@ -668,7 +683,9 @@ def capped_attention(out: torch.Tensor, q: torch.Tensor, key_cache: torch.Tensor
     tables = batch.block_tables
     _need(tables.dtype == torch.int32 and tables.is_contiguous() and tables.dim() == 2 and tables.shape[0] == n,
           "capped_attention: block tables")
-    _need(q.shape[1] == heads * dim and out.shape == (rows, heads * vdim) and out.is_contiguous()
+    out_stride = _rows(out, "out")
+    _need(q.shape[1] == heads * dim and out.shape == (rows, heads * vdim)
+          and (out_stride == heads * vdim or score_bias is None)
           and out.dtype == key_cache.dtype and key_cache.is_contiguous() and key_cache.dim() == 3
           and key_cache.shape[2] >= kv_heads * dim, "capped_attention: shapes")
     k_stride = key_cache.shape[2]
@@ -701,7 +718,7 @@ def capped_attention(out: torch.Tensor, q: torch.Tensor, key_cache: torch.Tensor
                 key_cache.shape[1], scale, int(window), _opt_ptr(work), _act(out), _stream(q)))
             return
         _check(lib.swm_masked_attention(
-            out.data_ptr(), q.data_ptr(), key_cache.data_ptr(), value_cache.data_ptr(), _opt_ptr(gate),
+            out.data_ptr(), out_stride, q.data_ptr(), key_cache.data_ptr(), value_cache.data_ptr(), _opt_ptr(gate),
             0 if gate is None else _rows(gate, "gate"), tables.data_ptr(), tables.shape[1], batch.q_start.data_ptr(),
             batch.ctx_len.data_ptr(), rows, n, longest, heads, kv_heads, dim, vdim, key_cache.shape[1], scale, softcap,
             int(window), int(chunk), 1 if sink else 0, k_stride, v_stride, _opt_ptr(work), _act(out), _stream(q)))
@@ -803,6 +820,147 @@ def latent_rope_cache(q_out: torch.Tensor, q_latent: torch.Tensor, q_rot: torch.
             rank, rot, _act(q_latent), _stream(q_out)))
 
 
+def embed_stream(stream: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, scale: float,
+                 rows_out: Optional[torch.Tensor] = None, weight: Optional[torch.Tensor] = None, offset: float = 0.0,
+                 eps: float = 0.0, out: Optional[torch.Tensor] = None) -> None:
+    """stream (fp32 [rows, width]) = scale * table[ids]; ``rows_out`` = the table's rows as they are (its dtype);
+    ``out`` = stream / rms(stream) * (offset + weight) in the table's dtype."""
+    _dev(stream, ids, table, rows_out, weight, out)
+    _f32c(stream, "stream")
+    rows, width = stream.shape
+    _need(ids.dtype == torch.int64 and ids.is_contiguous() and ids.numel() == rows and table.dim() == 2
+          and table.is_contiguous() and table.shape[1] == width, "embed_stream: ids and table")
+    for t in (rows_out, out):
+        _need(t is None or (t.shape == stream.shape and t.dtype == table.dtype and t.is_contiguous()), "embed_stream: outputs")
+    if out is not None:
+        _f32c(weight, "weight")
+        _need(weight.numel() == width, "embed_stream: norm weight")
+    with _on_device_of(stream):
+        _check(load_library().swm_embed_stream(
+            stream.data_ptr(), _opt_ptr(rows_out), ids.data_ptr(), table.data_ptr(), table.shape[0], scale, _opt_ptr(weight),
+            offset, eps, _opt_ptr(out), rows, width, _act(table), _stream(stream)))
+
+
+def stream_split(split: torch.Tensor, stream: torch.Tensor, a: Optional[torch.Tensor] = None,
+                 b: Optional[torch.Tensor] = None, c: Optional[torch.Tensor] = None) -> None:
+    """stream (fp32, in place) += a + b + c (a, b: bf16 2-D views; c: fp32); split (bf16 [rows, 2 * width]) = high | low
+    with high + low = the new stream to 16 bits of mantissa."""
+    _dev(split, stream, a, b, c)
+    _f32c(stream, "stream")
+    rows, width = stream.shape
+    _need(split.dtype == torch.bfloat16 and split.is_contiguous() and split.shape == (rows, 2 * width), "stream_split: split")
+    for t in (a, b):
+        _need(t is None or (t.shape == stream.shape and t.dtype == torch.bfloat16), "stream_split: addend")
+    if c is not None:
+        _f32c(c, "c")
+        _need(c.shape == stream.shape, "stream_split: fp32 addend")
+    with _on_device_of(stream):
+        _check(load_library().swm_stream_split(
+            stream.data_ptr(), _opt_ptr(a), 0 if a is None else _rows(a, "a"), _opt_ptr(b), 0 if b is None else _rows(b, "b"),
+            _opt_ptr(c), split.data_ptr(), rows, width, _stream(stream)))
+
+
+def _slots_ok(slot_mapping: torch.Tensor, rows: int) -> None:
+    _need(slot_mapping.dtype == torch.int64 and slot_mapping.numel() == rows and slot_mapping.is_contiguous(),
+          "slot_mapping must be int64 [rows]")
+
+
+def head_norm_cache(q_out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, eps: float, heads: int,
+                    kv_heads: int, dim: int, vdim: int, key_cache: torch.Tensor, value_cache: torch.Tensor,
+                    slot_mapping: torch.Tensor, q_weight: Optional[torch.Tensor] = None,
+                    k_weight: Optional[torch.Tensor] = None) -> None:
+    """q, k, v: column ranges of ONE projection output.  q_out fp32 = every query head over its root mean square (times
+    ``q_weight`` [dim]); the keys likewise and the values as they are go to the caches [pages, page, kv_heads * size]."""
+    _dev(q_out, q, k, v, key_cache, value_cache, slot_mapping, q_weight, k_weight)
+    _f32c(q_out, "q_out")
+    rows, stride = q.shape[0], _rows(q, "q")
+    _need(q.shape[1] == heads * dim and q_out.shape == q.shape and k.shape == (rows, kv_heads * dim)
+          and v.shape == (rows, kv_heads * vdim) and _rows(k, "k") == stride and _rows(v, "v") == stride
+          and k.dtype == q.dtype and v.dtype == q.dtype, "head_norm_cache: q, k, v must share rows, stride and dtype")
+    _need(key_cache.dtype == q.dtype and value_cache.dtype == q.dtype and key_cache.is_contiguous()
+          and value_cache.is_contiguous() and key_cache.shape[-1] == kv_heads * dim
+          and value_cache.shape[-1] == kv_heads * vdim
+          and key_cache.numel() // (kv_heads * dim) == value_cache.numel() // (kv_heads * vdim),
+          "head_norm_cache: cache shapes")
+    _slots_ok(slot_mapping, rows)
+    for w in (q_weight, k_weight):
+        if w is not None:
+            _f32c(w, "head norm weight")
+            _need(w.numel() == dim, "head_norm_cache: weights")
+    with _on_device_of(q):
+        _check(load_library().swm_head_norm_cache(
+            q_out.data_ptr(), q.data_ptr(), k.data_ptr(), v.data_ptr(), stride, _opt_ptr(q_weight), _opt_ptr(k_weight), eps,
+            key_cache.data_ptr(), value_cache.data_ptr(), slot_mapping.data_ptr(), rows, heads, kv_heads, dim, vdim, _act(q),
+            _stream(q)))
+
+
+def _turn(positions: torch.Tensor, inv_freq: Optional[torch.Tensor], rows: int) -> int:
+    """-> rotated coordinates of a rotation by positions * inv_freq (0: none)."""
+    if inv_freq is None or inv_freq.numel() == 0:
+        return 0
+    _f32c(inv_freq, "inv_freq")
+    _need(positions.dtype == torch.int64 and positions.numel() == rows and positions.is_contiguous(),
+          "positions must be int64 [rows]")
+    return 2 * inv_freq.numel()
+
+
+def latent_down(q_out: Optional[torch.Tensor], q_down: Optional[torch.Tensor], q_weight: Optional[torch.Tensor],
+                kv_down: torch.Tensor, kv_weight: torch.Tensor, eps: float, positions: torch.Tensor, inv_freq: torch.Tensor,
+                cache: torch.Tensor, slot_mapping: torch.Tensor, pair_halves: bool = False, amplitude: float = 1.0) -> None:
+    """q_down [rows, q_rank], kv_down [rows, rank + rot]: column ranges of ONE projection output.  q_out (their dtype) =
+    the normed query latent; cache [pages, page, rank + rot] row = the normed key latent | the turned key part."""
+    _dev(q_out, q_down, q_weight, kv_down, kv_weight, positions, inv_freq, cache, slot_mapping)
+    rows, stride = kv_down.shape[0], _rows(kv_down, "kv_down")
+    rot = _turn(positions, inv_freq, rows)
+    rank = kv_down.shape[1] - rot
+    _f32c(kv_weight, "kv_weight")
+    _slots_ok(slot_mapping, rows)
+    _need(rank > 0 and kv_weight.numel() == rank and cache.dtype == kv_down.dtype and cache.is_contiguous()
+          and cache.shape[-1] == rank + rot, "latent_down: key latent and cache")
+    q_rank = 0
+    if q_down is not None:
+        q_rank = q_down.shape[1]
+        _f32c(q_weight, "q_weight")
+        _need(q_down.shape[0] == rows and _rows(q_down, "q_down") == stride and q_down.dtype == kv_down.dtype
+              and q_weight.numel() == q_rank and q_out.shape == q_down.shape and q_out.is_contiguous()
+              and q_out.dtype == q_down.dtype, "latent_down: query latent")
+    with _on_device_of(kv_down):
+        _check(load_library().swm_latent_down(
+            _opt_ptr(q_out), _opt_ptr(q_down), q_rank, _opt_ptr(q_weight), kv_down.data_ptr(), rank, kv_weight.data_ptr(),
+            stride, eps, positions.data_ptr(), inv_freq.data_ptr() if rot else None, rot, 1 if pair_halves else 0, amplitude,
+            cache.data_ptr(), slot_mapping.data_ptr(), rows, _act(kv_down), _stream(kv_down)))
+
+
+def head_project(out: torch.Tensor, a: torch.Tensor, b: torch.Tensor, q_rot: Optional[torch.Tensor] = None,
+                 positions: Optional[torch.Tensor] = None, inv_freq: Optional[torch.Tensor] = None,
+                 pair_halves: bool = False, amplitude: float = 1.0, gate: Optional[torch.Tensor] = None) -> None:
+    """out [rows, heads, N (+ rot)] = b[h] a[t, h] per head (b [heads, N, K] contiguous; a [rows, heads, K]; out, a, q_rot:
+    strided views with contiguous last dimensions), times sigmoid(gate) with gate [rows, heads] or [rows, heads * N]
+    (a 2-D view); behind the N numbers the turned ``q_rot`` [rows, heads, rot].  out: a's dtype or fp32."""
+    _dev(out, a, b, q_rot, positions, inv_freq, gate)
+    rows, heads, K = a.shape
+    N = b.shape[1]
+    rot = 0
+    if q_rot is not None and q_rot.shape[2] > 0:
+        rot = _turn(positions, inv_freq, rows)
+        _need(q_rot.shape == (rows, heads, rot) and q_rot.stride(2) == 1 and q_rot.dtype == a.dtype,
+              "head_project: one frequency per rotated pair")
+    _need(b.shape == (heads, N, K) and b.is_contiguous() and b.dtype == a.dtype and a.stride(2) == 1
+          and out.shape == (rows, heads, N + rot) and out.stride(2) == 1 and out.dtype in (a.dtype, torch.float32),
+          "head_project: shapes")
+    per_head = 0
+    if gate is not None:
+        per_head = 1 if gate.shape == (rows, heads) else 0
+        _need((per_head or gate.shape == (rows, heads * N)) and gate.dtype == a.dtype, "head_project: gate")
+    with _on_device_of(out):
+        _check(load_library().swm_head_project(
+            out.data_ptr(), _act(out), out.stride(0), out.stride(1), a.data_ptr(), a.stride(0), a.stride(1), b.data_ptr(), N, K,
+            q_rot.data_ptr() if rot else None, q_rot.stride(0) if rot else 0, q_rot.stride(1) if rot else 0,
+            positions.data_ptr() if rot else None, inv_freq.data_ptr() if rot else None, rot, 1 if pair_halves else 0,
+            amplitude, _opt_ptr(gate), 0 if gate is None else _rows(gate, "gate"), per_head, rows, heads, _act(a),
+            _stream(out)))
+
+
 def gla(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay_pre: torch.Tensor,
         decay_bias: Optional[torch.Tensor], tau: float, q_scale: float, state: torch.Tensor, batch, heads: int,
         dim: int, vdim: int) -> None:
@@ -864,4 +1022,6 @@ ops = SimpleNamespace(expert_ffn=expert_ffn, ACT_GELU=ACT_GELU, ACT_RELU2=ACT_RE
     clamped_glu=clamped_glu, relu2=relu2, rope_cache=rope_cache, group_router=group_router, group_pairs=group_pairs,
     capped_attention=capped_attention, lightning=lightning, gated_stream_step=gated_stream_step, poly_norm=poly_norm,
     gate_mul=gate_mul, latent_rope_cache=latent_rope_cache, gla=gla, ACT_NONE=ACT_NONE, glu_rows=glu_rows,
-    group_norm_add=group_norm_add, causal_conv=causal_conv, gated_delta=gated_delta)
+    group_norm_add=group_norm_add, causal_conv=causal_conv, gated_delta=gated_delta, embed_stream=embed_stream,
+    stream_split=stream_split, head_norm_cache=head_norm_cache, latent_down=latent_down, head_project=head_project,
+    ROUTER_SOFTMAX=ROUTER_SOFTMAX, ROUTER_SOFTMAX_CHOSEN=ROUTER_SOFTMAX_CHOSEN)

@@ -152,6 +152,36 @@ _BOGETAR_PRESETS = {
     "bogetar-2k": (2048, 2, 16, 4, 32, 2, 1408),   # 2 experts of gate + up + down 1408 = the Llama stack's 2816
     "bogetar-4k": (4096, 2, 32, 8, 32, 2, 2816),
 }
+
+
+
+def _dovisun_preset(width: int, repeats: int, heads: int, kv_heads: int, ff: int, experts: int, top: int,
+                    expert_ff: int) -> dict:
+    """A Dovisun stack of layer sizes that resemble a served model's, ten layer runs per repeat of its one loop: a
+    latent-attention layer (a 384-wide query latent, a 192-wide key latent plus 64 rotated coordinates per token), a
+    block of two attention layers and a latent-attention layer that runs twice, and three layers behind it; dense
+    feed-forwards and routed experts in turn."""
+    d = width // heads
+    latent = {"heads": heads, "dim": d // 2, "rot_dim": 64, "vdim": d, "kv_rank": 192, "q_rank": 384,
+              "scale": (d // 2 + 64) ** -0.5,
+              "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    attn = {"heads": heads, "kv_heads": kv_heads, "dim": d, "vdim": d, "scale": d ** -0.5}
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "top": top}}
+    kinds = [(latent, dense), (attn, moe), (attn, dense), (latent, moe), (attn, dense), (latent, moe), (attn, None)]
+    layers = [{"type": "latent_attention" if m is latent else "attention", "mixer": dict(m), "mlp": f} for m, f in kinds]
+    from .model_executor.models.dovisun import normalize_config
+    return normalize_config({"architecture": "Dovisun", "embedding": {"scale": width ** 0.5}, "layers": layers,
+                             "loop": {"start": 1, "stop": 4, "times": repeats}, "logit_softcap": 30.0,
+                             "norm": {"eps": 1e-6}, "vocab": 32000, "width": width})
+
+
+_DOVISUN_PRESETS = {
+    # name: (width, passes of the block of three layers, heads, kv heads, feed-forward size, experts, top, expert ff);
+    # two passes make ten layer runs
+    "dovisun-2k": (2048, 2, 16, 4, 4224, 32, 2, 1408),   # up + down of 4224 = gate + up + down of 2816
+    "dovisun-4k": (4096, 2, 32, 8, 8448, 32, 2, 2816),
+}
 # Llama stacks of the same width, depth and active feed-forward size, to measure the above against
 MODEL_PRESETS.update({
     "llama-2k": dict(architecture="llama", vocab_size=32000, hidden_size=2048, num_hidden_layers=10,
@@ -216,6 +246,8 @@ class ModelConfig:
             return _lalasun_preset(*_LALASUN_PRESETS[name])
         if name in _BOGETAR_PRESETS:
             return _bogetar_preset(*_BOGETAR_PRESETS[name])
+        if name in _DOVISUN_PRESETS:
+            return _dovisun_preset(*_DOVISUN_PRESETS[name])
         cfg_path = os.path.join(model, "config.json")
         if os.path.isfile(cfg_path):
             with open(cfg_path) as f:
@@ -231,6 +263,9 @@ class ModelConfig:
                 return normalize_config(raw)
             if raw.get("architecture") == "Bogetar":
                 from .model_executor.models.bogetar import normalize_config
+                return normalize_config(raw)
+            if raw.get("architecture") == "Dovisun":
+                from .model_executor.models.dovisun import normalize_config
                 return normalize_config(raw)
             arch = (raw.get("architectures") or [""])[0].lower()
             raw["architecture"] = "opt" if "opt" in arch else "llama"

@@ -406,3 +406,79 @@ class LatentAttention(nn.Module):
         out = torch.empty(rows, H * self.vdim, dtype=q.dtype, device=q.device)
         _C.mixer_ops.gate_mul(out, up.transpose(0, 1), gate)
         return out
+
+
+class UnitHeadAttention(nn.Module):
+    """Causal softmax attention without positions, grouped query heads over a paged cache: every query and key head is
+    divided by its root mean square (no weight), score = (q . k) * scale, and (``sink``) the softmax's denominator has one
+    more term exp(0).  Keys are cached after their norm; caches are [pages, page, kv_heads * size].  Norms, scores,
+    weights and sums are fp32."""
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, eps: float, sink: bool = True) -> None:
+        super().__init__()
+        if heads % kv_heads != 0:
+            raise ValueError(f"{heads} query heads cannot share {kv_heads} key/value heads evenly")
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
+        self.scale, self.eps, self.sink = float(scale), eps, bool(sink)
+
+    def cache_shapes(self, block_size: int):
+        """Per page: keys, values."""
+        return [(block_size, self.kv_heads * self.dim), (block_size, self.kv_heads * self.vdim)]
+
+    def forward(self, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, key_cache: torch.Tensor, value_cache: torch.Tensor,
+                md: InputMetadata, out: torch.Tensor) -> None:
+        """q, k, v: column ranges of one projection output; out [rows, heads * vdim]: a 2-D view that is filled."""
+        q32 = torch.empty(q.shape[0], self.heads * self.dim, dtype=torch.float32, device=q.device)
+        _C.mixer_ops.head_norm_cache(q32, q, k, v, self.eps, self.heads, self.kv_heads, self.dim, self.vdim, key_cache,
+                                     value_cache, md.slot_mapping)
+        _C.mixer_ops.capped_attention(out, q32, key_cache, value_cache, None, md.ragged, self.heads, self.kv_heads,
+                                      self.dim, self.vdim, self.scale, sink=self.sink)
+
+
+class LatentQueryAttention(nn.Module):
+    """``LatentAttention`` whose queries come through a latent of their own (c_q = rms_norm(W_dq x) * w_q, q = W_uq c_q),
+    with the rotation on pairs (i, i + rot / 2), an amplitude on its cos and sin (YaRN) and one gate number per head.
+    The cache row, the shared key/value head and the place of the up-projections are LatentAttention's; the two
+    products per head are kernels of their own: U_k[h] with the rotation of the query's other coordinates beside it
+    (straight into the attention kernel's fp32 query rows), U_v[h] with the head's gate behind it (straight into the
+    caller's output row)."""
+
+    def __init__(self, heads: int, dim: int, rot: int, vdim: int, rank: int, q_rank: int, scale: float,
+                 inv_freq: torch.Tensor, amplitude: float, eps: float, dtype: torch.dtype) -> None:
+        super().__init__()
+        self.heads, self.dim, self.rot, self.vdim, self.rank, self.q_rank = heads, dim, rot, vdim, rank, q_rank
+        self.scale, self.eps, self.amplitude = float(scale), eps, float(amplitude)
+        assert 2 * inv_freq.numel() == rot
+        self.register_buffer("inv_freq", inv_freq.to(torch.float32).clone(), persistent=False)
+        self.query_norm = nn.Parameter(torch.ones(q_rank, dtype=torch.float32), requires_grad=False)
+        self.latent_norm = nn.Parameter(torch.ones(rank, dtype=torch.float32), requires_grad=False)
+        self.query_up = nn.Parameter(torch.zeros(heads * (dim + rot), q_rank, dtype=dtype), requires_grad=False)
+        self.key_up_t = nn.Parameter(torch.zeros(heads, rank, dim, dtype=dtype), requires_grad=False)     # U_k[h]^T
+        self.value_up = nn.Parameter(torch.zeros(heads, vdim, rank, dtype=dtype), requires_grad=False)    # U_v[h]
+
+    def cache_shapes(self, block_size: int):
+        return [(block_size, self.rank + self.rot)]
+
+    def load_up_projections(self, query_up: torch.Tensor, key_up: torch.Tensor, value_up: torch.Tensor) -> None:
+        """query_up [heads * (dim + rot), q_rank], key_up [heads * dim, rank], value_up [heads * vdim, rank], as a checkpoint
+        stores them ([out, in])."""
+        self.query_up.data.copy_(query_up)
+        self.key_up_t.data.copy_(key_up.view(self.heads, self.dim, self.rank).transpose(1, 2))
+        self.value_up.data.copy_(value_up.view(self.heads, self.vdim, self.rank))
+
+    def forward(self, q_down: torch.Tensor, kv_down: torch.Tensor, gate: torch.Tensor, positions: torch.Tensor,
+                cache: torch.Tensor, md: InputMetadata, out: torch.Tensor) -> None:
+        """q_down [rows, q_rank], kv_down [rows, rank + rot], gate [rows, heads]: column ranges of one projection output;
+        out [rows, heads * vdim]: a 2-D view that is filled."""
+        rows, H, width = q_down.shape[0], self.heads, self.rank + self.rot
+        c_q = torch.empty(rows, self.q_rank, dtype=q_down.dtype, device=q_down.device)
+        _C.mixer_ops.latent_down(c_q, q_down, self.query_norm.data, kv_down, self.latent_norm.data, self.eps, positions,
+                                 self.inv_freq, cache, md.slot_mapping, True, self.amplitude)
+        q = torch.mm(c_q, self.query_up.data.t()).unflatten(1, (H, self.dim + self.rot))
+        q32 = torch.empty(rows, H * width, dtype=torch.float32, device=q.device)
+        _C.mixer_ops.head_project(q32.unflatten(1, (H, width)), q[:, :, :self.dim], self.key_up_t.data, q[:, :, self.dim:],
+                                  positions, self.inv_freq, True, self.amplitude)
+        mixed = torch.empty(rows, H * self.rank, dtype=q.dtype, device=q.device)
+        _C.mixer_ops.capped_attention(mixed, q32, cache, None, None, md.ragged, H, 1, width, self.rank, self.scale)
+        _C.mixer_ops.head_project(out.unflatten(1, (H, self.vdim)), mixed.unflatten(1, (H, self.rank)), self.value_up.data,
+                                  gate=gate)

@@ -297,6 +297,69 @@ def scaled_rotary_frequencies(rot_dims: int, base: float, scaling: Optional[dict
     return torch.tensor(out, dtype=torch.float64).to(torch.float32)
 
 
+def yarn_rotary(rot_dims: int, base: float, scaling: Optional[dict] = None) -> Tuple[torch.Tensor, float]:
+    """-> (frequencies fp32 [rot_dims / 2], amplitude of cos and sin), f_i = base^(-2i / rot_dims), scaled as YaRN does it
+    (``scaling``: factor, original, fast, slow; None: plain frequencies, amplitude 1).  With turns(i) = original f_i /
+    2 pi, the pairs up to the one that turns ``fast`` times keep f, those from the one that turns ``slow`` times on get
+    f / factor, the pairs between them a mix that is linear in i (the two ends rounded outwards to whole pairs); the
+    amplitude is 0.1 ln(factor) + 1.  Worked out in double precision, rounded once."""
+    half = rot_dims // 2
+    plain = [float(base) ** (-2.0 * i / rot_dims) for i in range(half)]
+    if not scaling:
+        return torch.tensor(plain, dtype=torch.float64).to(torch.float32), 1.0
+    factor, original = float(scaling["factor"]), float(scaling["original"])
+
+    def pair_with_turns(turns: float) -> float:
+        return half * math.log(original / (2.0 * math.pi * turns)) / math.log(base)
+    first = max(math.floor(pair_with_turns(scaling["fast"])), 0)
+    last = min(math.ceil(pair_with_turns(scaling["slow"])), rot_dims - 1)
+    span = max(last - first, 0.001)
+    freqs = []
+    for i, f in enumerate(plain):
+        share = min(1.0, max(0.0, (i - first) / span))
+        freqs.append(f / factor * share + f * (1.0 - share))
+    return torch.tensor(freqs, dtype=torch.float64).to(torch.float32), 0.1 * math.log(factor) + 1.0
+
+
+class LoopInput(nn.Module):
+    """What a pass of a repeated block of layers reads: x <- W_x x + W_0 x_0, x the fp32 stream and x_0 = scale *
+    embedding rows.  The second product is the same in every pass of a step, so it is taken once (``start``), of the
+    unscaled rows -- they are exact in the activation dtype --, and the scale multiplies the product.  With bf16 weights
+    the stream goes through the first product as a pair of bf16 numbers (high | low, so the weight is kept twice side
+    by side) with fp32 accumulation and fp32 output: the stream is never rounded to bf16."""
+
+    def __init__(self, width: int, scale: float, dtype: torch.dtype) -> None:
+        super().__init__()
+        self.width, self.scale, self.dtype = width, float(scale), dtype
+        copies = 1 if dtype == torch.float32 else 2
+        self.stream_weight = nn.Parameter(torch.zeros(width, copies * width, dtype=dtype), requires_grad=False)
+        self.embed_weight = nn.Parameter(torch.zeros(width, width, dtype=dtype), requires_grad=False)
+
+    def load(self, weight: torch.Tensor) -> None:
+        """weight [width, 2 * width] = [W_x | W_0]."""
+        w = self.width
+        for lo in range(0, self.stream_weight.shape[1], w):
+            self.stream_weight.data[:, lo:lo + w].copy_(weight[:, :w])
+        self.embed_weight.data.copy_(weight[:, w:])
+
+    def start(self, rows: torch.Tensor) -> torch.Tensor:
+        """rows: the step's embedding rows, unscaled, in the activation dtype.  -> fp32 [rows, width]."""
+        if rows.dtype == torch.float32:
+            return torch.mm(rows, self.embed_weight.data.t())
+        return torch.mm(rows, self.embed_weight.data.t(), out_dtype=torch.float32)
+
+    def forward(self, stream: torch.Tensor, from_embedding: torch.Tensor, a: Optional[torch.Tensor] = None,
+                b: Optional[torch.Tensor] = None, c: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """stream += a + b + c in place (the outputs of the layer before), then -> the new stream of the pass."""
+        if self.dtype == torch.float32:
+            if a is not None or b is not None or c is not None:
+                _C.mixer_ops.stream_add_norm(stream, None, 0.0, 0.0, None, a, b, c)
+            return torch.addmm(from_embedding, stream, self.stream_weight.data.t(), beta=self.scale)
+        split = torch.empty(stream.shape[0], 2 * self.width, dtype=self.dtype, device=stream.device)
+        _C.mixer_ops.stream_split(split, stream, a, b, c)
+        return torch.addmm(from_embedding, split, self.stream_weight.data.t(), beta=self.scale, out_dtype=torch.float32)
+
+
 class ClampedGLU(nn.Module):
     """Gated activation with limits: x = gate | up;  g = min(gate, limit), u = clamp(up, -limit, limit);
     out = g * sigmoid(alpha * g) * (u + shift).  alpha = 1.702 makes g sigmoid(alpha g) the sigmoid form of gelu."""

@@ -11,7 +11,8 @@ routed sum so that the caller's residual add can take both.  The same layer, by 
 (``score="softmax"``: scores are the softmax over all experts), whose groups score their best expert
 (``group_score="max"``), whose weights are the chosen scores as they are (``normalize=False``) and whose experts have
 a gated hidden layer with limits (``activation="clamped_glu"``: g = min(gate x, limit), u = clamp(up x, +-limit),
-g sigmoid(alpha g) (u + 1)).
+g sigmoid(alpha g) (u + shift); alpha 1, no limit and shift 0 make it silu(g) u).  ``score="softmax_chosen"``: the choice
+goes by the logits and the weights are their softmax over the chosen ones (a ``router_bias`` is part of the logits).
 
 Rows are grouped by expert on the device (a stable sort of the (row, choice) pairs by expert id, then a binary
 search for every expert's first pair), so each expert's rows are one contiguous run and the host never waits.
@@ -82,21 +83,27 @@ class GroupRoutedExperts(nn.Module):
     def __init__(self, width: int, num_experts: int, top: int, ff: int, shared_ff: Optional[int], groups: int,
                  keep_groups: int, scale: float, dtype: torch.dtype, linear_method=None, score: str = "sigmoid",
                  group_score: str = "top2", normalize: bool = True, activation: str = "relu2",
-                 limit: float = float("inf"), glu_alpha: float = 1.702) -> None:
+                 limit: float = float("inf"), glu_alpha: float = 1.702, glu_shift: float = 1.0, router_bias: bool = False,
+                 router_dtype: torch.dtype = torch.float32) -> None:
         super().__init__()
-        if score not in ("sigmoid", "softmax") or group_score not in ("top2", "max") or \
+        if score not in ("sigmoid", "softmax", "softmax_chosen") or group_score not in ("top2", "max") or \
                 activation not in ("relu2", "clamped_glu"):
             raise ValueError(f"unknown router score {score!r}, group score {group_score!r} or activation {activation!r}")
         if activation == "clamped_glu" and shared_ff:
             raise NotImplementedError("a shared expert with a gated hidden layer")
-        self.softmax, self.group_best_one, self.normalize = score == "softmax", group_score == "max", bool(normalize)
-        self.glu = (float(glu_alpha), float(limit), 1.0) if activation == "clamped_glu" else None
+        self.softmax = {"sigmoid": 0, "softmax": _C.mixer_ops.ROUTER_SOFTMAX,
+                        "softmax_chosen": _C.mixer_ops.ROUTER_SOFTMAX_CHOSEN}[score]
+        self.group_best_one, self.normalize = group_score == "max", bool(normalize)
+        self.glu = (float(glu_alpha), float(limit), float(glu_shift)) if activation == "clamped_glu" else None
         if num_experts % groups != 0 or not (1 <= keep_groups <= groups) or keep_groups * (num_experts // groups) < top:
             raise ValueError(f"{num_experts} experts in {groups} groups with {keep_groups} kept cannot give {top} choices")
         self.width, self.num_experts, self.top, self.ff = width, num_experts, top, ff
         self.groups, self.keep_groups, self.scale = groups, keep_groups, float(scale)
-        # the router is fp32 whatever the model's dtype
-        self.router = nn.Parameter(torch.zeros(num_experts, width, dtype=torch.float32), requires_grad=False)
+        # the router's products are fp32 whatever the model's dtype; a checkpoint's bf16 router may be kept as it is
+        # (``router_dtype``): its products with bf16 inputs are exact in fp32
+        self.router = nn.Parameter(torch.zeros(num_experts, width, dtype=router_dtype), requires_grad=False)
+        self.router_bias = nn.Parameter(torch.zeros(num_experts, dtype=torch.float32), requires_grad=False) \
+            if router_bias else None
         self.correction = nn.Parameter(torch.zeros(num_experts, dtype=torch.float32), requires_grad=False)
         # a gated hidden layer: gate and up rows in runs of 16, as the fused kernel reads them (``mixer_ops.glu_rows``)
         self.up = nn.Parameter(torch.empty(num_experts, 32 * (-(-ff // 16)) if self.glu else ff, width, dtype=dtype),
@@ -107,15 +114,25 @@ class GroupRoutedExperts(nn.Module):
             self.shared_up = ColumnParallelLinear(width, shared_ff, False, dtype, linear_method)
             self.shared_down = RowParallelLinear(shared_ff, width, False, dtype, linear_method)
 
+    def router_logits(self, h: torch.Tensor) -> torch.Tensor:
+        """fp32 [rows, experts]: products and sums in fp32 (the library's GEMM; no reduced-precision matrix mode is switched
+        on)."""
+        w = self.router.data.t()
+        if w.dtype == h.dtype and h.dtype != torch.float32:
+            if self.router_bias is None:
+                return torch.mm(h, w, out_dtype=torch.float32)
+            return torch.addmm(self.router_bias.data, h, w, out_dtype=torch.float32)
+        if self.router_bias is None:
+            return torch.matmul(h.float(), w)
+        return torch.addmm(self.router_bias.data, h.float(), w)
+
     def forward(self, h: torch.Tensor) -> Tuple[Optional[torch.Tensor], torch.Tensor]:
         """-> (shared expert's output in h's dtype or None, routed experts' weighted sum in fp32)."""
-        # fp32 products with the fp32 router (the library's GEMM; no reduced-precision matrix mode is switched on)
-        logits = torch.matmul(h.float(), self.router.data.t())
-        chosen, weights = _C.mixer_ops.group_router(logits, self.correction.data, self.top, self.groups,
+        out = torch.empty(h.shape[0], self.width, dtype=torch.float32, device=h.device)
+        chosen, weights = _C.mixer_ops.group_router(self.router_logits(h), self.correction.data, self.top, self.groups,
                                                     self.keep_groups, self.scale, self.softmax, self.group_best_one,
-                                                    self.normalize)
+                                                    self.normalize, clear=out)
         order, start = group_pairs_by_expert(chosen, self.num_experts)
-        out = torch.zeros(h.shape[0], self.width, dtype=torch.float32, device=h.device)
         _C.mixer_ops.expert_ffn(out, h, self.up.data, self.down.data, order, start, self.top, 1.0,
                                 activation=_C.mixer_ops.ACT_RELU2, pair_weight=weights, glu=self.glu)
         shared = None
@@ -127,7 +144,9 @@ class GroupRoutedExperts(nn.Module):
         return shared, out
 
     def load_named(self, w: Dict[str, torch.Tensor]) -> None:
-        self.router.data.copy_(w["router"].float())
+        self.router.data.copy_(w["router"])
+        if self.router_bias is not None:
+            self.router_bias.data.copy_(w["router.b"].float())
         if "correction" in w:
             self.correction.data.copy_(w["correction"].float())
         if self.glu:

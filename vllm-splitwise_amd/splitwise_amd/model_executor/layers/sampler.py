@@ -161,10 +161,18 @@ class FollowerSamples:
 
 
 class Sampler(nn.Module):
-    def __init__(self, vocab_size: int, org_vocab_size: Optional[int] = None) -> None:
+    def __init__(self, vocab_size: int, org_vocab_size: Optional[int] = None,
+                 logit_softcap: Optional[float] = None) -> None:
         super().__init__()
         self.vocab_size = vocab_size
         self.org_vocab_size = org_vocab_size or vocab_size
+        self.logit_softcap = float(logit_softcap) if logit_softcap else None
+
+    def cap_logits(self, logits: torch.Tensor) -> torch.Tensor:
+        """fp32 cap * tanh(logits / cap) for a model that bounds its logits; otherwise the logits as they are."""
+        if self.logit_softcap is None:
+            return logits
+        return torch.tanh(logits.float() / self.logit_softcap).mul_(self.logit_softcap)
 
     def _get_logits(self, hidden_states: torch.Tensor, embedding: torch.Tensor,
                     embedding_bias: Optional[torch.Tensor]) -> torch.Tensor:
@@ -176,7 +184,7 @@ class Sampler(nn.Module):
         from ..parallel_state import tensor_model_parallel_gather
         logits = tensor_model_parallel_gather(logits, dst=0)
         if logits is not None:
-            logits = logits[:, :self.org_vocab_size]           # drop the padding of the sharded vocabulary
+            logits = self.cap_logits(logits[:, :self.org_vocab_size])      # without the padding of the sharded vocabulary
         return logits
 
     def forward(self, embedding: torch.Tensor, hidden_states: torch.Tensor,

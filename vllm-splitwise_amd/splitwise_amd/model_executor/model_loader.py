@@ -14,6 +14,7 @@ import torch.nn as nn
 
 from ..config import ModelConfig
 from .models.bogetar import BogetarForCausalLM
+from .models.dovisun import DovisunForCausalLM
 from .models.lalasun import LalasunForCausalLM
 from .models.lapilorn import LapilornForCausalLM
 from .models.llama import LlamaForCausalLM
@@ -21,7 +22,8 @@ from .models.nepevik import NepevikForCausalLM
 from .models.opt import OPTForCausalLM
 
 _ARCH = {"llama": LlamaForCausalLM, "opt": OPTForCausalLM, "nepevik": NepevikForCausalLM,
-         "lapilorn": LapilornForCausalLM, "lalasun": LalasunForCausalLM, "bogetar": BogetarForCausalLM}
+         "lapilorn": LapilornForCausalLM, "lalasun": LalasunForCausalLM, "bogetar": BogetarForCausalLM,
+         "dovisun": DovisunForCausalLM}
 
 
 def architecture_class(name: str):
