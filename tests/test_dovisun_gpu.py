@@ -1,0 +1,534 @@
+"""Dovisun on the GPU against the plain statement in ``oracle/dovisun.py``: every mechanism alone, then whole models
+through the engine -- the stream after every layer run, whole prompts, token-by-token decoding, portions down to two
+tokens, mixed batches, pages that are reused, greedy generation through ``LLM.generate``, the replay entry point.
+
+The models are small and random (``tests/dovisun_util.py``); where random numbers would hide a fault (one far key among
+hundreds, a key on a page border, a missing softmax sink, a choice that only the router's bias makes) the inputs are
+built so that it shows.
+"""
+import random
+from types import SimpleNamespace
+
+import pytest
+import torch
+
+import dovisun_util as du
+from mixer_harness import DEV, attention_case, ops, paged, ragged, steps_of, tol_of
+from oracle import dovisun as oracle
+
+pytestmark = pytest.mark.gpu
+F64 = torch.float64
+BOTH = [torch.float32, torch.bfloat16]
+
+
+# ------------------------------------------------------------------ the stream
+@pytest.mark.parametrize("dtype", BOTH)
+@pytest.mark.parametrize("width", [22, 48, 200, 1030, 2560])
+def test_embedding_starts_the_stream(dtype, width):
+    g = torch.Generator().manual_seed(width)
+    table = torch.randn(31, width, generator=g).to(dtype)
+    table[7] *= 1e-4                                                     # a row small enough for eps to count
+    ids = torch.tensor([0, 30, 7, 7, 12])
+    w = torch.randn(width, generator=g) * 0.3 + 1.0
+    for want_rows, want_norm in [(True, True), (False, True), (True, False), (False, False)]:
+        stream = torch.full((5, width), float("nan"), device=DEV)
+        rows = torch.zeros(5, width, dtype=dtype, device=DEV) if want_rows else None
+        out = torch.zeros(5, width, dtype=dtype, device=DEV) if want_norm else None
+        ops().embed_stream(stream, ids.to(DEV), table.to(DEV), 2.75, rows, w.to(DEV) if want_norm else None, 0.0, 1e-5, out)
+        want = 2.75 * table[ids].double()
+        torch.testing.assert_close(stream.cpu().double(), want, atol=1e-6, rtol=1e-6)
+        if want_rows:
+            assert torch.equal(rows.cpu(), table[ids])
+        if want_norm:
+            torch.testing.assert_close(out.cpu().double(), oracle.rms_norm(want, w.double(), 1e-5), **tol_of(dtype))
+
+
+def test_an_id_beyond_the_table_shows():
+    table = torch.randn(5, 16).to(DEV)
+    stream = torch.empty(3, 16, device=DEV)
+    ops().embed_stream(stream, torch.tensor([4, 5, -1], device=DEV), table, 1.0)
+    assert torch.isfinite(stream[0]).all() and torch.isnan(stream[1:]).all()
+
+
+@pytest.mark.parametrize("width", [22, 48, 1030, 2560])
+def test_stream_as_a_pair_of_bf16_numbers(width):
+    g = torch.Generator().manual_seed(width)
+    rows = 6
+    x = torch.randn(rows, width, generator=g) * 10
+    y = torch.randn(rows, 2 * width + 3, generator=g).bfloat16()
+    a, b, c = y[:, 3:3 + width], y[:, 3 + width:], torch.randn(rows, width, generator=g)
+    for use in [(1, 0, 1), (1, 1, 1), (1, 0, 0), (0, 0, 1), (0, 0, 0)]:
+        stream, split = x.clone().to(DEV), torch.empty(rows, 2 * width, dtype=torch.bfloat16, device=DEV)
+        ops().stream_split(split, stream, *(t.to(DEV) if u else None for t, u in zip((a, b, c), use)))
+        want = x.double() + sum(t.double() for t, u in zip((a, b, c), use) if u)
+        torch.testing.assert_close(stream.cpu().double(), want, atol=1e-5, rtol=1e-6)
+        s = split.cpu().double()
+        assert torch.equal(split[:, :width].cpu(), stream.cpu().bfloat16())
+        assert ((s[:, :width] + s[:, width:] - stream.cpu().double()).abs() <= 2.0 ** -16 * stream.cpu().double().abs() + 1e-30).all()
+
+
+@pytest.mark.parametrize("dtype", BOTH)
+@pytest.mark.parametrize("rows,width", [(1, 48), (5, 22), (70, 128), (33, 1000)])
+def test_input_of_a_pass(rows, width, dtype):
+    """x <- W_x x + W_0 (scale * row), the layer's outputs added to x before; bf16 weights do not round the stream."""
+    from splitwise_amd.model_executor.layers.basic import LoopInput
+    g = torch.Generator().manual_seed(rows)
+    w = (torch.randn(width, 2 * width, generator=g) * width ** -0.5).bfloat16()
+    e = torch.randn(rows, width, generator=g).bfloat16()
+    x = torch.randn(rows, width, generator=g) * 5
+    a, c = torch.randn(rows, width, generator=g).bfloat16(), torch.randn(rows, width, generator=g)
+    loop = LoopInput(width, 3.5, dtype).to(DEV)
+    loop.load(w.to(dtype).to(DEV))
+    base = loop.start(e.to(dtype).to(DEV))
+    for use in (True, False):
+        stream = x.clone().to(DEV)
+        got = loop(stream, base, a.to(dtype).to(DEV) if use else None, None, c.to(DEV) if use else None)
+        want_x = x.double() + (a.double() + c.double() if use else 0.0)
+        torch.testing.assert_close(stream.cpu().double(), want_x, atol=2e-6, rtol=1e-6)
+        want = torch.cat([want_x, 3.5 * e.double()], -1) @ w.double().T
+        assert got.dtype == torch.float32
+        assert (got.cpu().double() - want).abs().max() < 6e-5 * want.abs().max()
+
+
+@pytest.mark.parametrize("dtype", BOTH)
+@pytest.mark.parametrize("ff,lead,extra", [(40, 8, 16), (33, 5, 2), (2112, 0, 64), (64, 4, 8)])
+def test_relu_squared_into_a_wider_row(dtype, ff, lead, extra):
+    g = torch.Generator().manual_seed(ff)
+    src = torch.randn(9, lead + ff + 8, generator=g).to(dtype)
+    dst = torch.full((9, ff + extra), 7.0, dtype=dtype, device=DEV)
+    ops().relu2(dst[:, :ff], src.to(DEV)[:, lead:lead + ff])
+    torch.testing.assert_close(dst[:, :ff].cpu().double(), torch.relu(src[:, lead:lead + ff].double()).pow(2), **tol_of(dtype))
+    assert (dst[:, ff:] == 7.0).all()                                    # the neighbours in the row are untouched
+
+
+# ------------------------------------------------------------------ attention without positions
+@pytest.mark.parametrize("H,G,d,dv", [(4, 2, 16, 12), (3, 1, 7, 5), (3, 3, 24, 24), (8, 2, 64, 72), (2, 2, 130, 258), (1, 1, 512, 2)])
+@pytest.mark.parametrize("dtype", BOTH)
+@pytest.mark.parametrize("weighted", [False, True])
+def test_head_norm_and_cache_write(H, G, d, dv, dtype, weighted):
+    g = torch.Generator().manual_seed(H * 100 + d)
+    rows, page, lead = 7, 8, 2 if d % 2 == 0 else 3
+    proj = torch.randn(rows, lead + H * d + G * (d + dv) + 1, generator=g).to(dtype)
+    if d % 2 == 0:
+        proj = proj[:, :-1].contiguous()                                 # even rows: the two-at-a-time path
+    cut = [lead, lead + H * d, lead + H * d + G * d, lead + H * d + G * (d + dv)]
+    proj[3, cut[0]:cut[0] + d] *= 1e-3                                   # a query small enough for eps to count
+    q, k, v = (proj[:, lo:hi] for lo, hi in zip(cut, cut[1:]))
+    slots = torch.tensor([9, -1, 17, 31, 16, 8, 0])
+    kc, vc = torch.full((4, page, G * d), 5.0, dtype=dtype), torch.full((4, page, G * dv), 5.0, dtype=dtype)
+    kd, vd, pd = kc.to(DEV), vc.to(DEV), proj.to(DEV)
+    wq, wk = (torch.randn(d, generator=g) for _ in range(2)) if weighted else (None, None)
+    q_out = torch.full((rows, H * d), float("nan"), device=DEV)
+    ops().head_norm_cache(q_out, *(pd[:, lo:hi] for lo, hi in zip(cut, cut[1:])), 1e-5, H, G, d, dv, kd, vd, slots.to(DEV),
+                          wq.to(DEV) if weighted else None, wk.to(DEV) if weighted else None)
+
+    def unit(x, w):
+        u = oracle.rms_unit(x.double(), 1e-5)
+        return u * w.double() if weighted else u
+    torch.testing.assert_close(q_out.cpu().double().view(rows, H, d), unit(q.view(rows, H, d), wq), atol=2e-5, rtol=2e-5)
+    kf, vf = kd.cpu().view(-1, G, d), vd.cpu().view(-1, G, dv)
+    for t, slot in enumerate(slots.tolist()):
+        if slot >= 0:
+            torch.testing.assert_close(kf[slot].double(), unit(k[t].view(G, d), wk), **tol_of(dtype))
+            assert torch.equal(vf[slot], v[t].view(G, dv))
+    rest = [s for s in range(32) if s not in slots.tolist()]
+    assert (kf[rest] == 5.0).all() and (vf[rest] == 5.0).all()           # the row without a slot wrote nowhere
+
+
+@pytest.mark.parametrize("H,G,d,dv,page", [(4, 2, 16, 12, 16), (3, 1, 7, 5, 8), (6, 6, 8, 24, 16), (8, 2, 64, 32, 16), (6, 2, 20, 40, 32),
+                                           (16, 1, 24, 72, 16)])
+@pytest.mark.parametrize("mode", ["prompt", "decode", "pairs", "portions"])
+@pytest.mark.parametrize("dtype", BOTH)
+def test_unit_head_attention_with_a_sink(H, G, d, dv, page, mode, dtype):
+    """The attention kernel over normed heads: keys far away, on both sides of a page border and of a 32-key tile, the
+    query's own key, the sequence's first key; a query that meets only keys of the opposite direction, so that the sink
+    takes nearly everything; the output written into a column range of a wider row."""
+    n = 300
+    last = n - 1
+    spikes = [(last, 2, 0), (last - 1, page - 1, H - 1), (last - 2, page, 0), (last - 3, 31, H - 1), (last - 4, 32, 0),
+              (last - 5, last - 5, H - 1), (100, 0, 0), (129, 127, H - 1), (128, 128, 0), (40, 39, H - 1), (last - 45, 0, H - 1)]
+    q, k, v = attention_case(H, G, d, dv, n, spikes, seed=H * 1000 + d)
+    q, k = oracle.rms_unit(q.double(), 1e-6), oracle.rms_unit(k.double(), 1e-6)
+    q[7] = -k[:8].mean(0).repeat_interleave(H // G, 0) * 3
+    kc, vc, table = paged(k.reshape(n, -1), v.reshape(n, -1), page, dtype, seed=d)
+    kk = torch.stack([kc.cpu().double()[table[t // page], t % page].view(G, d) for t in range(n)])
+    vv = torch.stack([vc.cpu().double()[table[t // page], t % page].view(G, dv) for t in range(n)])
+    scale = 9.0 / d                                                      # aligned heads score 9: e^9 outweighs 300 others
+    want = oracle.causal_attention(q, kk, vv, scale, sink=True).reshape(n, H * dv)
+    no_sink = oracle.causal_attention(q[:9], kk, vv, scale).reshape(9, H * dv)
+    assert (no_sink - want[:9]).abs().max() > 0.05                       # the test would not notice a missing sink otherwise
+    seqs, rows = steps_of(mode, n, table)
+    batch = ragged(seqs)
+    qd = q[rows].reshape(len(rows), H * d).float().contiguous().to(DEV)
+    wide = torch.full((len(rows), H * dv + 9), 3.0, dtype=dtype, device=DEV)
+    ops().capped_attention(wide[:, 5:5 + H * dv], qd, kc, vc, None, batch, H, G, d, dv, scale, sink=True)
+    tol = dict(atol=3e-5, rtol=3e-5) if dtype == torch.float32 else dict(atol=2e-2, rtol=2e-2)
+    torch.testing.assert_close(wide[:, 5:5 + H * dv].cpu().double(), want[rows], **tol)
+    assert (wide[:, :5] == 3.0).all() and (wide[:, 5 + H * dv:] == 3.0).all()
+
+
+@pytest.mark.parametrize("dtype", BOTH)
+def test_keys_shared_among_workgroups_into_a_wider_row(dtype):
+    """Decode steps of few sequences with long contexts and many query heads per key: the join launch writes the column
+    range too, and takes the sink once."""
+    n, page, H, d, dv = 1500, 16, 16, 24, 40
+    rows = [n - 1, 1201, 700]
+    q, k, v = attention_case(H, 1, d, dv, n, [(n - 1, 3, 0), (1201, 650, H - 1), (700, 699, 5)], seed=7)
+    kc, vc, table = paged(k.reshape(n, d), v.reshape(n, dv), page, dtype, seed=5)
+    kk = torch.stack([kc.cpu().double()[table[t // page], t % page].view(1, d) for t in range(n)])
+    vv = torch.stack([vc.cpu().double()[table[t // page], t % page].view(1, dv) for t in range(n)])
+    want = torch.stack([oracle.causal_attention(q[t:t + 1].double(), kk, vv, 0.9, sink=True, first_position=t)[0] for t in rows])
+    wide = torch.full((3, H * dv + 6), 3.0, dtype=dtype, device=DEV)
+    from splitwise_amd import _C_mixers
+    assert _C_mixers.load_library().swm_masked_attention_workspace_floats(3, 3, 1, H, 1, dv, page, len(table), 0, 0) > 0
+    ops().capped_attention(wide[:, :H * dv], q[rows].reshape(3, H * d).contiguous().to(DEV), kc, vc, None,
+                           ragged([(t, 1, 0, table) for t in rows]), H, 1, d, dv, 0.9, sink=True)
+    tol = dict(atol=3e-5, rtol=3e-5) if dtype == torch.float32 else dict(atol=2e-2, rtol=2e-2)
+    torch.testing.assert_close(wide[:, :H * dv].cpu().double(), want.reshape(3, H * dv), **tol)
+    assert (wide[:, H * dv:] == 3.0).all()
+
+
+# ------------------------------------------------------------------ latent attention
+@pytest.mark.parametrize("rank,q_rank,rot", [(20, 14, 4), (8, 0, 2), (64, 48, 16), (130, 33, 6), (12, 5, 0), (192, 384, 64)])
+@pytest.mark.parametrize("dtype", BOTH)
+@pytest.mark.parametrize("halves,amplitude", [(True, 1.1386), (True, 1.0), (False, 1.07)])
+def test_both_latents_of_a_row(rank, q_rank, rot, dtype, halves, amplitude):
+    from oracle import lalasun
+    g = torch.Generator().manual_seed(rank)
+    rows, page = 8, 8
+    positions = torch.tensor([0, 1, 7, 8, 9, 300, 2047, 70000])
+    proj = torch.randn(rows, 3 + q_rank + rank + rot, generator=g).to(dtype)
+    qd, kd = proj[:, 3:3 + q_rank], proj[:, 3 + q_rank:]
+    proj[6] *= 1e-3                                                      # latents small enough for eps to count
+    wq, wk = torch.randn(max(q_rank, 1), generator=g) * 0.3 + 1.0, torch.randn(rank, generator=g) * 0.3 + 1.0
+    f = oracle.yarn_frequencies({"dims": rot, "base": 30.0, "scaling": du.yarn()}) if rot else []
+    slots = torch.tensor([9, 0, 17, 31, -1, 8, 2, 5])
+    cache = torch.full((4, page, rank + rot), 5.0, dtype=dtype, device=DEV)
+    q_out = torch.empty(rows, q_rank, dtype=dtype, device=DEV) if q_rank else None
+    pd = proj.to(DEV)
+    inv = torch.tensor(f, dtype=torch.float32, device=DEV)
+    ops().latent_down(q_out, pd[:, 3:3 + q_rank] if q_rank else None, wq.to(DEV) if q_rank else None, pd[:, 3 + q_rank:],
+                      wk.to(DEV), 1e-5, positions.to(DEV), inv, cache, slots.to(DEV), halves, amplitude)
+    if q_rank:
+        torch.testing.assert_close(q_out.cpu().double(), oracle.rms_norm(qd.double(), wq.double(), 1e-5), **tol_of(dtype))
+    flat = cache.cpu().view(-1, rank + rot).double()
+    for t, slot in enumerate(slots.tolist()):
+        if slot < 0:
+            continue
+        torch.testing.assert_close(flat[slot, :rank], oracle.rms_norm(kd[t, :rank].double(), wk.double(), 1e-5), **tol_of(dtype))
+        y = kd[t:t + 1, rank:].double()
+        turned = oracle.rotate_halves(y, int(positions[t]), f, amplitude) if halves else \
+            amplitude * lalasun.rotate_neighbours(y, int(positions[t]), f)
+        torch.testing.assert_close(flat[slot, rank:], turned[0], **tol_of(dtype))
+    assert (flat[[s for s in range(32) if s not in slots.tolist()]] == 5.0).all()
+
+
+@pytest.mark.parametrize("H,N,K,rot", [(3, 20, 8, 4), (2, 64, 64, 0), (4, 192, 64, 64), (5, 7, 13, 2), (1, 130, 72, 8), (2, 40, 200, 6)])
+@pytest.mark.parametrize("rows", [1, 33, 150])
+@pytest.mark.parametrize("dtype,out_dtype", [(torch.float32, torch.float32), (torch.bfloat16, torch.float32), (torch.bfloat16, torch.bfloat16)])
+def test_product_per_head(H, N, K, rot, rows, dtype, out_dtype):
+    """With the rotation of the other coordinates beside it; with a gate per head and per channel behind it; from and into
+    strided rows."""
+    g = torch.Generator().manual_seed(N * 10 + K)
+    src = torch.randn(rows, H * (K + rot), generator=g).to(dtype)
+    b = (torch.randn(H, N, K, generator=g) * K ** -0.5).to(dtype)
+    positions = torch.randint(0, 5000, (rows,), generator=g)
+    f = oracle.yarn_frequencies({"dims": rot, "base": 30.0}) if rot else []
+    heads = src.unflatten(1, (H, K + rot))
+    sd = src.to(DEV).unflatten(1, (H, K + rot))
+    want = torch.stack([heads[:, h, :K].double() @ b[h].double().T for h in range(H)], 1)
+    tol = dict(atol=3e-5, rtol=3e-5) if out_dtype == torch.float32 else dict(atol=3e-2, rtol=2e-2)
+    out = torch.full((rows, H * (N + rot)), float("nan"), dtype=out_dtype, device=DEV)
+    ops().head_project(out.unflatten(1, (H, N + rot)), sd[:, :, :K], b.to(DEV), sd[:, :, K:], positions.to(DEV),
+                       torch.tensor(f, dtype=torch.float32, device=DEV), True, 1.2)
+    got = out.cpu().double().view(rows, H, N + rot)
+    torch.testing.assert_close(got[:, :, :N], want, **tol)
+    for t in range(0, rows, 7):
+        torch.testing.assert_close(got[t, :, N:], oracle.rotate_halves(heads[t, :, K:].double(), int(positions[t]), f, 1.2), **tol)
+    wide_gate = torch.randn(rows, H * N + 5, generator=g).to(dtype)
+    for gate in (wide_gate[:, 2:2 + H], wide_gate[:, 3:3 + H * N]):
+        wide = torch.full((rows, H * N + 11), 3.0, dtype=out_dtype, device=DEV)
+        ops().head_project(wide[:, 7:7 + H * N].unflatten(1, (H, N)), sd[:, :, :K], b.to(DEV),
+                           gate=wide_gate.to(DEV)[:, 2:2 + H] if gate.shape[1] == H else wide_gate.to(DEV)[:, 3:3 + H * N])
+        s = torch.sigmoid(gate.double())
+        s = s.unsqueeze(-1) if gate.shape[1] == H else s.view(rows, H, N)
+        torch.testing.assert_close(wide[:, 7:7 + H * N].cpu().double(), (want * s).reshape(rows, -1), **tol)
+        assert (wide[:, :7] == 3.0).all() and (wide[:, 7 + H * N:] == 3.0).all()
+
+
+@pytest.mark.parametrize("mode", ["prompt", "decode", "pairs", "portions"])
+@pytest.mark.parametrize("H,dim,rot,vdim,rank,q_rank,page", [(3, 8, 4, 12, 20, 14, 16), (4, 32, 16, 64, 128, 48, 16), (6, 12, 6, 10, 33, 9, 8)])
+def test_latent_attention_layer(mode, H, dim, rot, vdim, rank, q_rank, page):
+    """The whole layer from the three projections to the gated heads, fp32, with scores so peaked that single far keys
+    carry the output (asserted), over shuffled pages and in every cut."""
+    from splitwise_amd.model_executor.layers.attention import LatentQueryAttention
+    g = torch.Generator().manual_seed(rank)
+    n, eps = 300, 1e-5
+    m = {"heads": H, "dim": dim, "rot_dim": rot, "vdim": vdim, "kv_rank": rank, "scale": 1.0,
+         "rot": {"dims": rot, "base": 200.0, "scaling": du.yarn(4.0, 128, 16.0, 1.0)}}
+    width = q_rank + rank + rot + H
+    h = torch.randn(n, width, generator=g)                               # "projections" that pick columns of the input
+    eye = torch.eye(width)
+    w = {"dq": eye[:q_rank], "dkv": eye[q_rank:q_rank + rank + rot], "g": eye[q_rank + rank + rot:],
+         "dq.norm": torch.randn(q_rank, generator=g) * 0.3 + 1.0, "dkv.norm": torch.randn(rank, generator=g) * 0.3 + 1.0,
+         "uq": torch.randn(H * (dim + rot), q_rank, generator=g) * 3 * q_rank ** -0.5,
+         "uk": torch.randn(H * dim, rank, generator=g) * 2 * (rank * dim) ** -0.5, "uv": torch.randn(H * vdim, rank, generator=g) * rank ** -0.5,
+         "o": torch.eye(H * vdim)}
+    want = oracle.latent_attention_mixer(h.double(), {k: v.double() for k, v in w.items()}, m, eps)
+    freqs = torch.tensor(oracle.yarn_frequencies(m["rot"]), dtype=torch.float32)
+    layer = LatentQueryAttention(H, dim, rot, vdim, rank, q_rank, 1.0, freqs, oracle.yarn_amplitude(m["rot"]), eps, torch.float32)
+    layer.query_norm.data.copy_(w["dq.norm"])
+    layer.latent_norm.data.copy_(w["dkv.norm"])
+    layer.load_up_projections(w["uq"], w["uk"], w["uv"])
+    layer = layer.to(DEV)
+    pages = -(-n // page)
+    table = list(range(pages + 3))
+    random.Random(rank).shuffle(table)
+    table = table[:pages]
+    cache = torch.full((pages + 3, page, rank + rot), float("nan"), device=DEV)
+    slot_of = torch.tensor([table[t // page] * page + t % page for t in range(n)])
+
+    def run(batch, rows):
+        x = h[rows].to(DEV)
+        out = torch.empty(len(rows), H * vdim, device=DEV)
+        md = SimpleNamespace(ragged=batch, slot_mapping=slot_of[rows].to(DEV))
+        layer(x[:, :q_rank], x[:, q_rank:q_rank + rank + rot], x[:, q_rank + rank + rot:], torch.tensor(rows, device=DEV), cache, md, out)
+        return out.cpu().double()
+    got = run(ragged([(0, n, 0, table)]), list(range(n)))                # fills the cache
+    torch.testing.assert_close(got, want, atol=2e-4, rtol=2e-4)
+    seqs, rows = steps_of(mode, n, table)
+    torch.testing.assert_close(run(ragged(seqs), rows), want[rows], atol=2e-4, rtol=2e-4)
+    # single far keys carry rows: without the keys before the middle, late rows come out otherwise by far
+    late = oracle.latent_attention_mixer(torch.cat([torch.zeros(150, width), h[150:]]).double(), {k: v.double() for k, v in w.items()}, m, eps)
+    assert ((late - want)[200:].abs().amax(-1) > 0.2).float().mean() > 0.5
+
+
+# ------------------------------------------------------------------ router and experts
+@pytest.mark.parametrize("experts,top", [(5, 2), (8, 1), (12, 12), (64, 6), (256, 8), (1, 1)])
+def test_router_with_a_bias_and_a_softmax_over_the_chosen(experts, top):
+    g = torch.Generator().manual_seed(experts)
+    rows, width = 37, 20
+    z = torch.randn(rows, experts, generator=g) * 2
+    z[5] *= 60                                     # a softmax over all would underflow beyond the best: the choice goes by logits
+    out = torch.full((rows, width), 9.0, device=DEV)
+    chosen, weights = ops().group_router(z.to(DEV), None, top, 1, 1, 1.0, ops().ROUTER_SOFTMAX_CHOSEN, clear=out)
+    assert (out == 0).all()
+    best, want = torch.topk(z.double(), top, dim=-1)
+    assert torch.equal(chosen.cpu().long(), want)
+    torch.testing.assert_close(weights.cpu().double(), torch.softmax(best, -1), atol=1e-6, rtol=1e-5)
+
+
+@pytest.mark.parametrize("dtype,width,ff,experts,top", [
+    (torch.float32, 48, 24, 5, 2), (torch.bfloat16, 48, 24, 5, 2), (torch.bfloat16, 64, 96, 8, 1), (torch.float32, 22, 9, 7, 3),
+    (torch.bfloat16, 22, 9, 7, 7), (torch.bfloat16, 128, 32, 4, 4), (torch.float32, 40, 17, 3, 1)])
+def test_routed_experts(dtype, width, ff, experts, top):
+    from splitwise_amd.model_executor.layers.moe import GroupRoutedExperts
+    g = torch.Generator().manual_seed(width + ff)
+    rows = 77
+    w = {}
+    for e in range(experts):
+        w[f"e{e}.gate"], w[f"e{e}.up"] = (((torch.randn(ff, width, generator=g) * 2 * width ** -0.5)).to(dtype) for _ in range(2))
+        w[f"e{e}.down"] = (torch.randn(width, ff, generator=g) * 2 * ff ** -0.5).to(dtype)
+    w["router"], w["router.b"] = torch.randn(experts, width, generator=g).bfloat16().to(dtype), torch.randn(experts, generator=g)
+    h = torch.randn(rows, width, generator=g).to(dtype)
+    layer = GroupRoutedExperts(width, experts, top, ff, None, 1, 1, 1.0, dtype, None, score="softmax_chosen",
+                               activation="clamped_glu", glu_alpha=1.0, glu_shift=0.0, router_bias=True, router_dtype=dtype)
+    layer.load_named(w)
+    layer = layer.to(DEV)
+    torch.testing.assert_close(layer.router_logits(h.to(DEV)).cpu().double(), h.double() @ w["router"].double().T + w["router.b"].double(),
+                               atol=2e-5, rtol=2e-5)
+    shared, got = layer(h.to(DEV))
+    wd = {k: v.double() for k, v in w.items()}
+    want = oracle.moe_ff(h.double(), wd, {"router": {"top": top}})
+    assert shared is None and got.dtype == torch.float32
+    assert (got.cpu().double() - want).abs().max() < (2e-5 if dtype == torch.float32 else 2e-2) * want.abs().max()
+    if top < experts:                              # the bias decides some choices
+        free = oracle.route(h.double(), wd["router"], 0 * wd["router.b"], top)[0]
+        assert not torch.equal(free, oracle.route(h.double(), wd["router"], wd["router.b"], top)[0])
+
+
+# --------------------------------------------------------------- whole models through the engine
+FP32_TOL = 2e-4
+
+
+@pytest.fixture(scope="module")
+def models(tmp_path_factory):
+    out = {}
+    for name, (make, seed) in du.MODELS.items():
+        cfg = make()
+        sd = du.random_weights(cfg, seed)
+        path = du.write_model(str(tmp_path_factory.mktemp("dovisun_" + name)), cfg, sd)
+        g = torch.Generator().manual_seed(seed)
+        reqs = {f"r{i}": torch.randint(0, cfg["vocab"], (n,), generator=g).tolist()
+                for i, n in enumerate([70, 41, 18, 1, 33, 52, 150])}
+        out[name] = SimpleNamespace(cfg=cfg, sd=sd, path=path, reqs=reqs,
+                                    want={rid: oracle.logits(cfg, sd, toks, dtype=F64) for rid, toks in reqs.items()})
+    return out
+
+
+@pytest.fixture(scope="module")
+def engines(models):
+    cache = {}
+
+    def get(name, dtype, **kw):
+        key = (name, dtype, tuple(sorted(kw.items())))
+        if key not in cache:
+            cache[key] = du.make_engine(models[name].path, dtype, **kw)
+        return cache[key]
+    return get
+
+
+@pytest.mark.parametrize("name", sorted(du.MODELS))
+def test_stream_after_every_layer_run(models, engines, name):
+    m = models[name]
+    engine = engines(name, "float32")
+    model = engine.model_executor.driver_worker.model_runner.model
+    toks = m.reqs["r4"]
+    _, want = oracle.logits(m.cfg, m.sd, toks, dtype=F64, keep_streams=True)
+    model.keep_residuals = []
+    try:
+        du.Replayer(engine, {"r4": toks}).run_alone("r4", [len(toks)])
+        got = [r.cpu().double() for r in model.keep_residuals]
+    finally:
+        model.keep_residuals = None
+    assert len(got) == len(want) == len(oracle.layer_runs(m.cfg))
+    for i, (a, b) in enumerate(zip(got, want)):
+        assert (a - b).abs().max() < 1e-4 * b.abs().max(), f"run {i}"
+
+
+@pytest.mark.parametrize("name", sorted(du.MODELS))
+def test_whole_prompts_match_the_plain_statement(models, engines, name):
+    m = models[name]
+    for rid, toks in m.reqs.items():
+        got = du.Replayer(engines(name, "float32"), {rid: toks}).run_alone(rid, [len(toks)])
+        assert du.row_error(got, m.want[rid]) < FP32_TOL, rid
+
+
+@pytest.mark.parametrize("name", sorted(du.MODELS))
+def test_decoding_token_by_token(models, engines, name):
+    """Most of a prompt at once and then 45 (and 100) tokens one by one, and a sequence fed one token at a time from its
+    very first."""
+    m = models[name]
+    for rid, first in (("r0", 25), ("r6", 50)):
+        toks = m.reqs[rid]
+        got = du.Replayer(engines(name, "float32"), {rid: toks}).run_alone(rid, [first] + [1] * (len(toks) - first))
+        assert du.row_error(got, m.want[rid]) < FP32_TOL
+    toks = m.reqs["r2"]
+    got = du.Replayer(engines(name, "float32"), {"r2": toks}).run_alone("r2", [1] * len(toks))
+    assert du.row_error(got, m.want["r2"]) < FP32_TOL
+
+
+@pytest.mark.parametrize("name", sorted(du.MODELS))
+@pytest.mark.parametrize("portions", [[2] * 35, [3, 2, 16, 1, 2, 7, 17, 2, 2, 18], [15, 1, 16, 17, 2, 19], [33, 31, 2, 4]])
+def test_portions_of_prompts(models, engines, name, portions):
+    m = models[name]
+    toks = m.reqs["r0"]
+    assert sum(portions) == len(toks)
+    got = du.Replayer(engines(name, "float32"), {"r0": toks}).run_alone("r0", portions)
+    assert du.row_error(got, m.want["r0"]) < FP32_TOL
+
+
+@pytest.mark.parametrize("name,dtype,tol", [(n, "float32", FP32_TOL) for n in sorted(du.MODELS)] + [("e", "bfloat16", 0.08)])
+def test_mixed_batches_reuse_pages_and_slots(models, engines, name, dtype, tol):
+    """Six unequal requests over three places and a pool of 9 pages: portions beside single tokens, requests that sit out
+    steps, pages handed on as requests end.  Every request must come out as it does alone."""
+    m = models[name]
+    reqs = {r: t for r, t in m.reqs.items() if r != "r6"}
+    engine = engines(name, dtype, max_tokens=144, max_requests=3)
+    rp = du.Replayer(engine, reqs)
+    free_before = engine.scheduler.block_manager.get_num_free_gpu_blocks()
+    steps = [{"r0": 3, "r2": 16}, {"r0": 16, "r2": 1, "r3": 1}, {"r0": 2, "r1": 29, "r2": 1}, {"r0": 17, "r1": 2},
+             {"r0": 30, "r1": 1}, {"r1": 9, "r0": 1}, {"r0": 1, "r4": 20}]
+    for step in steps:
+        rp.step(step)
+    rnd = random.Random(7)
+    pending = ["r5"]
+    while any(rp.at[r] < len(reqs[r]) for r in reqs):
+        live = [r for r in rp.live if rp.at[r] < len(reqs[r])]
+        while pending and len(live) < 3:
+            nxt = pending[0]
+            need = -(-len(reqs[nxt]) // 16)
+            held = sum(-(-len(reqs[r]) // 16) for r in live)
+            if held + need > 9:
+                break
+            live.append(pending.pop(0))
+        step = {}
+        for r in live:
+            left = len(reqs[r]) - rp.at[r]
+            step[r] = min(left, rnd.choice([1, 1, 2, 3, 16, 21]))
+        if rnd.random() < 0.3 and len(step) > 1:
+            step.pop(rnd.choice(sorted(step)))                  # somebody sits this step out
+        rp.step(step)
+    for rid in reqs:
+        assert du.row_error(rp.result(rid), m.want[rid]) < tol, rid
+    assert engine.scheduler.block_manager.get_num_free_gpu_blocks() == free_before
+    assert engine.scheduler.state_slots.num_free() == 3
+
+
+def test_bfloat16_is_close_and_does_not_depend_on_the_cut(models, engines):
+    """On a model whose routers choose all their experts, so that nothing discrete can fall the other way."""
+    m = models["e"]
+    toks = m.reqs["r0"]
+    whole = du.Replayer(engines("e", "bfloat16"), {"r0": toks}).run_alone("r0", [len(toks)])
+    cut = du.Replayer(engines("e", "bfloat16"), {"r0": toks}).run_alone("r0", [2, 3, 16, 1, 1, 30, 17])
+    assert du.row_error(whole, m.want["r0"]) < 0.08
+    assert du.row_error(cut, m.want["r0"]) < 0.08
+    assert du.row_error(cut, whole) < 0.05
+
+
+@pytest.mark.parametrize("name", sorted(du.MODELS))
+def test_greedy_generation_through_the_entry_point(models, name):
+    """``LLM.generate`` with the scheduler's own policy: a token budget of 16 cuts the prompts into portions that run
+    beside other requests' decoded tokens.  Every generated token must be (within rounding) the arg-max of the plain
+    statement's logits for the text before it, and its log-probability that of the soft-capped logits."""
+    from splitwise_amd import LLM, SamplingParams
+    m = models[name]
+    llm = LLM(model=m.path, dtype="float32", block_size=16, max_model_len=128, max_num_seqs=3,
+              max_num_batched_tokens=16, num_gpu_blocks_override=20, swap_space=0, enforce_eager=True)
+    prompts = [m.reqs["r1"], m.reqs["r2"], m.reqs["r3"], m.reqs["r4"][:20]]
+    outs = llm.generate(prompt_token_ids=prompts, sampling_params=SamplingParams(temperature=0.0, max_tokens=12, logprobs=1,
+                                                                                 ignore_eos=True))
+    assert len(outs) == len(prompts)
+    for prompt, out in zip(prompts, outs):
+        new = out.outputs[0].token_ids
+        assert len(new) == 12
+        full = oracle.logits(m.cfg, m.sd, list(prompt) + list(new), dtype=F64)
+        for k, tok in enumerate(new):
+            row = full[len(prompt) + k - 1]
+            assert row[tok] >= row.max() - 1e-3 * (row.max() - row.min()), (k, tok, int(row.argmax()))
+            lp = out.outputs[0].logprobs[k][tok]
+            assert abs(float(getattr(lp, "logprob", lp)) - float(torch.log_softmax(row, -1)[tok])) < 2e-3
+    sched = llm.llm_engine.scheduler
+    assert sched.state_slots.num_free() == 3 and not sched.running and not sched.waiting
+
+
+def test_trace_run_replays_a_schedule(models, tmp_path):
+    """``bin/trace_run`` as a user starts it: steps on standard input, ``done <step>`` after each, logits files in the
+    order of the entries; requests that sit out a step, end, and hand their pages on."""
+    import json
+    import os
+    import subprocess
+    import numpy as np
+    m = models["b"]
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    a, b, c = m.reqs["r1"], m.reqs["r2"], m.reqs["r4"]
+    steps = [
+        {"step": 0, "entries": [{"id": "a", "tokens": a[:7], "want": [0, 6]}, {"id": "b", "tokens": b[:2], "want": []}], "end": []},
+        {"step": 1, "entries": [{"id": "b", "tokens": b[2:], "want": [15]}, {"id": "a", "tokens": a[7:8], "want": [0]}], "end": ["b"]},
+        {"step": 2, "entries": [{"id": "a", "tokens": a[8:], "want": [len(a) - 9]}, {"id": "c", "tokens": c, "want": [0, len(c) - 1]}],
+         "end": ["a", "c"]},
+        {"step": 3, "entries": [{"id": "b", "tokens": b, "want": [len(b) - 1]}], "end": ["b"]},        # the name comes back
+    ]
+    out = tmp_path / "out"
+    proc = subprocess.run([os.path.join(root, "bin", "trace_run"), "--model", m.path, "--dtype", "float32", "--out", str(out),
+                           "--max-tokens", "128", "--max-requests", "2"],
+                          input="".join(json.dumps(s) + "\n" for s in steps), capture_output=True, text=True, timeout=300)
+    assert proc.returncode == 0, proc.stderr[-2000:]
+    assert [l for l in proc.stdout.splitlines() if l.startswith("done")] == [f"done {i}" for i in range(4)]
+    vocab = m.cfg["vocab"]
+    want = {0: [m.want["r1"][0], m.want["r1"][6]], 1: [m.want["r2"][17], m.want["r1"][7]],
+            2: [m.want["r1"][len(a) - 1], m.want["r4"][0], m.want["r4"][len(c) - 1]], 3: [m.want["r2"][len(b) - 1]]}
+    for step, rows in want.items():
+        got = torch.from_numpy(np.fromfile(out / f"{step}.f32", dtype="<f4").reshape(-1, vocab))
+        assert got.shape[0] == len(rows)
+        assert du.row_error(got, torch.stack(rows)) < FP32_TOL, step
