@@ -1,7 +1,8 @@
 // Tuning harness for the int4 GEMMs (not part of the shipped library): compiles quant_gemm.hip with its
 // experiment knobs switched on, times back-to-back launches with HIP events and compares every variant with the
 // first one run on the same inputs.
-//   hipcc -O3 -std=c++17 --offload-arch=gfx950 -DSW_QUANT_EXPERIMENT -I include -I vllm-splitwise_amd/csrc \
+//   hipcc -O3 -std=c++17 --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops \
+//         -DSW_QUANT_EXPERIMENT -I include -I vllm-splitwise_amd/csrc \
 //         tools/quant_exp.hip -o gpurun_out/quant_exp
 //   SW_QUANT_WAVES=4 SW_QUANT_TMT=4 gpurun_out/quant_exp 256 13824 5120
 #include "../vllm-splitwise_amd/csrc/quant_gemm.hip"
