@@ -82,12 +82,12 @@ def test_input_of_a_pass(rows, width, dtype):
     base = loop.start(e.to(dtype).to(DEV))
     for use in (True, False):
         stream = x.clone().to(DEV)
-        got = loop(stream, base, a.to(dtype).to(DEV) if use else None, None, c.to(DEV) if use else None)
+        got = loop(stream, a.to(dtype).to(DEV) if use else None, None, c.to(DEV) if use else None)
         want_x = x.double() + (a.double() + c.double() if use else 0.0)
         torch.testing.assert_close(stream.cpu().double(), want_x, atol=2e-6, rtol=1e-6)
         want = torch.cat([want_x, 3.5 * e.double()], -1) @ w.double().T
-        assert got.dtype == torch.float32
-        assert (got.cpu().double() - want).abs().max() < 6e-5 * want.abs().max()
+        assert got.dtype == base.dtype == torch.float32
+        assert (got.cpu().double() + base.cpu().double() - want).abs().max() < 6e-5 * want.abs().max()
 
 
 @pytest.mark.parametrize("dtype", BOTH)

@@ -29,37 +29,68 @@ __device__ __forceinline__ void rotation_of(const RotationParams& p, int64_t row
 
 constexpr int kLdThreads = 256;
 
-// one workgroup per row
-template <typename T>
+// A wave per latent of a row: the even wave of a pair norms the query latent (or has nothing to do), the odd one norms the
+// key latent, turns the key part and writes both into the cache.  V: neighbours per access (2: sizes, strides and bases
+// are even); a latent of up to 512 numbers stays in registers between its sum and its scaling.
+template <typename T, int V>
+__device__ __forceinline__ void norm_latent(void* __restrict__ out, int64_t out_at, const void* __restrict__ in, int64_t at,
+                                            int size, const float* __restrict__ weight, float eps) {
+  using S = typename Conv<T>::store_t;
+  struct alignas(V * sizeof(S)) Piece { S x[V]; };
+  constexpr int PER = 512 / 64 / V;
+  const int lane = threadIdx.x & 63;
+  const S* src = static_cast<const S*>(in) + at;
+  S* dst = static_cast<S*>(out) + out_at;
+  auto get = [&](int c) { return *reinterpret_cast<const Piece*>(src + c); };
+  Piece held[PER];
+  float ss = 0.0f;
+  auto add = [&](const Piece& p) {
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      const float x = Conv<T>::to_float(p.x[e]);
+      ss += x * x;
+    }
+  };
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int c = (lane + 64 * j) * V;
+    if (c < size) {
+      held[j] = get(c);
+      add(held[j]);
+    }
+  }
+  for (int c = (lane + 64 * PER) * V; c < size; c += 64 * V) add(get(c));
+  const float f = 1.0f / sqrtf(sw::wave_sum(ss) / (float)size + eps);
+  auto put = [&](int c, const Piece& p) {
+    Piece o;
+#pragma unroll
+    for (int e = 0; e < V; ++e) o.x[e] = Conv<T>::from_float(Conv<T>::to_float(p.x[e]) * f * weight[c + e]);
+    *reinterpret_cast<Piece*>(dst + c) = o;
+  };
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int c = (lane + 64 * j) * V;
+    if (c < size) put(c, held[j]);
+  }
+  for (int c = (lane + 64 * PER) * V; c < size; c += 64 * V) put(c, get(c));
+}
+
+template <typename T, int V>
 __global__ __launch_bounds__(kLdThreads) void latent_down_kernel(
     void* __restrict__ q_out, const void* __restrict__ q_down, int q_rank, const float* __restrict__ q_weight,
     const void* __restrict__ kv_down, int rank, const float* __restrict__ kv_weight, int64_t in_stride, float eps,
-    RotationParams turn, void* __restrict__ cache, const int64_t* __restrict__ slot_mapping) {
-  __shared__ float red[16];
-  const int64_t t = blockIdx.x, in = t * in_stride;
-  float ssq = 0.0f, ssk = 0.0f;
-  for (int c = threadIdx.x; c < q_rank; c += kLdThreads) {
-    const float v = ld<T>(q_down, in + c);
-    ssq += v * v;
+    RotationParams turn, void* __restrict__ cache, const int64_t* __restrict__ slot_mapping, int64_t rows) {
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int64_t t = (int64_t)blockIdx.x * (kLdThreads / 128) + (wave >> 1), in = t * in_stride;
+  if (t >= rows) return;                                     // no barrier below
+  if ((wave & 1) == 0) {
+    if (q_rank > 0) norm_latent<T, V>(q_out, t * (int64_t)q_rank, q_down, in, q_rank, q_weight, eps);
+    return;
   }
-  for (int c = threadIdx.x; c < rank; c += kLdThreads) {
-    const float v = ld<T>(kv_down, in + c);
-    ssk += v * v;
-  }
-  ssq = block_sum(ssq, red);
-  ssk = block_sum(ssk, red);
-  if (q_rank > 0) {
-    const float f = 1.0f / sqrtf(ssq / (float)q_rank + eps);
-    for (int c = threadIdx.x; c < q_rank; c += kLdThreads)
-      st<T>(q_out, t * (int64_t)q_rank + c, ld<T>(q_down, in + c) * f * q_weight[c]);
-  }
-  const int64_t slot = slot_mapping[t];                      // uniform over the workgroup
+  const int64_t slot = slot_mapping[t];
   if (slot < 0) return;
-  const float f = 1.0f / sqrtf(ssk / (float)rank + eps);
   const int64_t dst = slot * (int64_t)(rank + turn.rot);
-  for (int c = threadIdx.x; c < rank; c += kLdThreads)
-    st<T>(cache, dst + c, ld<T>(kv_down, in + c) * f * kv_weight[c]);
-  for (int i = threadIdx.x; i < turn.rot / 2; i += kLdThreads) {
+  for (int i = lane; i < turn.rot / 2; i += 64) {
     int u, v;
     float c, s;
     rotation_of(turn, t, i, &u, &v, &c, &s);
@@ -67,6 +98,7 @@ __global__ __launch_bounds__(kLdThreads) void latent_down_kernel(
     st<T>(cache, dst + rank + u, a * c - b * s);
     st<T>(cache, dst + rank + v, b * c + a * s);
   }
+  norm_latent<T, V>(cache, dst, kv_down, in, rank, kv_weight, eps);
 }
 
 // What a head_project launch reads and writes besides the tile loop's operands.
@@ -166,9 +198,22 @@ int swm_latent_down(void* q_out, const void* q_down, int q_rank, const float* q_
                    (rot == 0 || (positions != nullptr && inv_freq != nullptr)),
                "latent_down: a part is missing");
   const RotationParams turn{positions, inv_freq, rot, pair_halves, amplitude};
-  SWM_DISPATCH_ACT(act_dtype, hipLaunchKernelGGL(latent_down_kernel<T>, dim3((unsigned)rows), dim3(kLdThreads), 0,
-                                                 static_cast<hipStream_t>(stream), q_out, q_down, q_rank, q_weight, kv_down,
-                                                 rank, kv_weight, in_stride, eps, turn, cache, slot_mapping););
+  const uintptr_t piece = act_dtype == SW_F32 ? 8 : 4;
+  auto even = [&](const void* p) { return reinterpret_cast<uintptr_t>(p) % piece == 0; };
+  const bool pairs = q_rank % 2 == 0 && rank % 2 == 0 && in_stride % 2 == 0 && even(q_out) && even(q_down) &&
+                     even(kv_down) && even(cache);
+  const int per = kLdThreads / 128;
+  const dim3 grid((unsigned)((rows + per - 1) / per));
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (pairs) {
+    SWM_DISPATCH_ACT(act_dtype, hipLaunchKernelGGL((latent_down_kernel<T, 2>), grid, dim3(kLdThreads), 0, s, q_out, q_down,
+                                                   q_rank, q_weight, kv_down, rank, kv_weight, in_stride, eps, turn, cache,
+                                                   slot_mapping, rows););
+  } else {
+    SWM_DISPATCH_ACT(act_dtype, hipLaunchKernelGGL((latent_down_kernel<T, 1>), grid, dim3(kLdThreads), 0, s, q_out, q_down,
+                                                   q_rank, q_weight, kv_down, rank, kv_weight, in_stride, eps, turn, cache,
+                                                   slot_mapping, rows););
+  }
   SW_CHECK_LAUNCH();
   return SW_OK;
 }

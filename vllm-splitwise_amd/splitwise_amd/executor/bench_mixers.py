@@ -1,4 +1,4 @@
-"""Throughput of a Nepevik (or Lapilorn, Lalasun or Bogetar) stack beside a Llama stack of the same width, depth and active feed-forward size
+"""Throughput of a Nepevik (or Lapilorn, Lalasun, Bogetar or Dovisun) stack beside a Llama stack of the same width, depth and active feed-forward size
 (random weights), and every mixer kernel beside the like kernel of the Llama path with their distances from
 the roofline.  ``bench.py --mixers`` prints the result as one JSON line.
 
@@ -676,15 +676,175 @@ def kernel_table_bogetar(width: int = 2048, heads: int = 16, kv_heads: int = 4, 
     return rows
 
 
+@torch.inference_mode()
+def kernel_table_dovisun(width: int = 2048, heads: int = 16, kv_heads: int = 4, prefill_rows: int = 4096,
+                         decode_seqs: int = 64, decode_ctx: int = 2047, rank: int = 192, q_rank: int = 384, rot: int = 64,
+                         ff: int = 4224, experts: int = 32, top: int = 2, expert_ff: int = 1408) -> List[dict]:
+    """The kernels of the Dovisun layers beside their like: attention with a sink beside the same kernel without; unit heads
+    with their cache write beside the rotation kernel behind a per-head norm (Bogetar's); latent attention beside Lalasun's
+    (same rows, no window), and the two products per head with what is fused to them beside Lalasun's batched library
+    product + layout kernel; the norm of both latents beside the layout kernel's norm; the stream's steps beside the fused add
+    + norm; relu^2 beside the gated unit; the router and the experts beside Bogetar's."""
+    from .. import _C
+    ops = _C.mixer_ops
+    dev, bf = torch.device("cuda"), torch.bfloat16
+    d, page = width // heads, 16
+    dim, vdim, row = d // 2, d, rank + rot
+    rows: List[dict] = []
+    for phase, seqs in (("prefill", [(0, prefill_rows // 2, 0, None), (0, prefill_rows // 2, 1, None)]),
+                        ("decode", [(decode_ctx, 1, i, None) for i in range(decode_seqs)])):
+        total_pages, laid = 0, []
+        for ctx, n, slot, _ in seqs:
+            pages = -(-(ctx + n) // page)
+            laid.append((ctx, n, slot, list(range(total_pages, total_pages + pages))))
+            total_pages += pages
+        batch = _ragged(laid, dev)
+        T = sum(s[1] for s in laid)
+        pairs = sum(i + 1 for c, n, _, _ in laid for i in range(c, c + n))
+        keys = sum(c + n for c, n, _, _ in laid)
+        pos = torch.cat([torch.arange(c, c + n) for c, n, _, _ in laid]).to(dev)
+        slots = torch.cat([torch.tensor([tb[p // page] * page + p % page for p in range(c, c + n)])
+                           for c, n, _, tb in laid]).to(dev)
+        # ---------------------------------------------------------------- attention on unit heads
+        kc = torch.randn(total_pages, page, kv_heads * d, device=dev).to(bf)
+        vc = torch.randn(total_pages, page, kv_heads * d, device=dev).to(bf)
+        q = torch.randn(T, heads * d, device=dev)
+        both = torch.empty(T, ff + heads * d, dtype=bf, device=dev)
+        abytes = keys * kv_heads * d * 2 * 2 + T * heads * d * (4 + 2)
+        for name, kw, like in (("attention with a sink (causal, into a wider row)", dict(sink=True), ""),
+                               ("capped_attention as Lapilorn runs it (causal, no cap)", {}, "attention with a sink")):
+            out = both[:, ff:] if kw else torch.empty(T, heads * d, dtype=bf, device=dev)
+            t = _time(lambda: ops.capped_attention(out, q, kc, vc, None, batch, heads, kv_heads, d, d, d ** -0.5, **kw))
+            rows.append(_row(name, phase, t, abytes, 4.0 * pairs * heads * d, VALU_F32, like=like))
+        proj = torch.randn(T, (heads + 2 * kv_heads) * d, device=dev).to(bf)
+        cols = (proj[:, :heads * d], proj[:, heads * d:(heads + kv_heads) * d], proj[:, (heads + kv_heads) * d:])
+        q32, wq = torch.empty(T, heads * d, device=dev), torch.ones(d, device=dev)
+        nbytes = T * ((heads + 2 * kv_heads) * d * 2 + heads * d * 4 + 2 * kv_heads * d * 2)
+        t = _time(lambda: ops.head_norm_cache(q32, *cols, 1e-6, heads, kv_heads, d, d, kc, vc, slots))
+        rows.append(_row("head_norm_cache (unit heads)", phase, t, nbytes, 4.0 * T * heads * d, VALU_F32))
+        t = _time(lambda: ops.rope_cache(q32, *cols, pos, torch.zeros(0, device=dev), heads, kv_heads, d, d, kc, vc, slots, True, wq,
+                                         wq, 1e-6))
+        rows.append(_row("Bogetar rope_cache behind a per-head norm, nothing rotated", phase, t, nbytes, 4.0 * T * heads * d, VALU_F32,
+                         like="head_norm_cache"))
+        # ---------------------------------------------------------------- latent attention
+        lc = torch.randn(total_pages, page, row, device=dev).to(bf)
+        ql = torch.randn(T, heads * row, device=dev)
+        mixed = torch.empty(T, heads * rank, dtype=bf, device=dev)
+        t = _time(lambda: ops.capped_attention(mixed, ql, lc, None, None, batch, heads, 1, row, rank, d ** -0.5))
+        rows.append(_row("latent attention (one %d-wide row per token, as Lalasun's without a window)" % row, phase, t,
+                         keys * row * 2 + T * heads * (row * 4 + rank * 2), 2.0 * pairs * heads * (row + rank), VALU_F32))
+        down = torch.randn(T, q_rank + row + heads, device=dev).to(bf)
+        w_q, w_kv, inv = torch.ones(q_rank, device=dev), torch.ones(rank, device=dev), torch.rand(rot // 2, device=dev)
+        c_q = torch.empty(T, q_rank, dtype=bf, device=dev)
+        q_cols, kv_cols = down[:, :q_rank], down[:, q_rank:q_rank + row]
+        t = _time(lambda: ops.latent_down(c_q, q_cols, w_q, kv_cols, w_kv, 1e-6, pos, inv, lc, slots, True, 1.1))
+        rows.append(_row("latent_down (both latents normed, key part turned, cache write)", phase, t, T * (q_rank + row) * 2 * 2,
+                         4.0 * T * (q_rank + row), VALU_F32))
+        qh = torch.randn(T, heads * (dim + rot), device=dev).to(bf).unflatten(1, (heads, dim + rot))
+        ku_t = torch.randn(heads, rank, dim, device=dev).to(bf)
+        ku = ku_t.transpose(1, 2).contiguous()
+        vu = torch.randn(heads, vdim, rank, device=dev).to(bf)
+        vu_t = vu.transpose(1, 2).contiguous()
+        pbytes = T * heads * ((dim + rot) * 2 + row * 4) + heads * rank * dim * 2
+        pflops = 2.0 * T * heads * rank * dim
+        qv, q_plain, q_turn = ql.unflatten(1, (heads, row)), qh[:, :, :dim], qh[:, :, dim:]
+        t = _time(lambda: ops.head_project(qv, q_plain, ku_t, q_turn, pos, inv, True, 1.1))
+        rows.append(_row("head_project (queries into the latent, rotation beside)", phase, t, pbytes, pflops, MFMA_BF16))
+
+        def lalasun_queries():
+            lat = torch.bmm(qh[:, :, :dim].transpose(0, 1), ku)
+            ops.latent_rope_cache(ql, lat.transpose(0, 1), qh[:, :, dim:], down[:, q_rank:q_rank + row], w_kv, 1e-6, pos, inv, lc, slots)
+        t = _time(lalasun_queries)
+        rows.append(_row("Lalasun: batched library product + latent_rope_cache (norm and cache write in it)", phase, t,
+                         pbytes + T * row * 2 * 2, pflops, MFMA_BF16, like="head_project (queries)"))
+        gate = torch.randn(T, heads * vdim, device=dev).to(bf)
+        heads_out = both[:, ff:ff + heads * vdim].unflatten(1, (heads, vdim))
+        vbytes = T * heads * (rank + vdim) * 2 + heads * rank * vdim * 2
+        mixed_heads, head_gate = mixed.unflatten(1, (heads, rank)), gate[:, :heads]
+        t = _time(lambda: ops.head_project(heads_out, mixed_heads, vu, gate=head_gate))
+        rows.append(_row("head_project (heads out of the latent, gate behind)", phase, t, vbytes + T * heads * 2,
+                         2.0 * T * heads * rank * vdim, MFMA_BF16))
+        gated = torch.empty(T, heads * vdim, dtype=bf, device=dev)
+
+        def lalasun_values():
+            up = torch.bmm(mixed.unflatten(1, (heads, rank)).transpose(0, 1), vu_t)
+            ops.gate_mul(gated, up.transpose(0, 1), gate)
+        t = _time(lalasun_values)
+        rows.append(_row("Lalasun: batched library product + gate_mul", phase, t, vbytes + T * heads * vdim * 2,
+                         2.0 * T * heads * rank * vdim, MFMA_BF16, like="head_project (heads)"))
+        # ---------------------------------------------------------------- the stream
+        stream, hout = torch.randn(T, width, device=dev), torch.empty(T, width, dtype=bf, device=dev)
+        wn, a, c32 = torch.ones(width, device=dev), torch.randn(T, width, device=dev).to(bf), torch.randn(T, width, device=dev)
+        table = torch.randn(32000, width, device=dev).to(bf)
+        ids, raw = torch.randint(0, 32000, (T,), device=dev), torch.empty(T, width, dtype=bf, device=dev)
+        x0 = torch.empty(T, width, device=dev)
+        t = _time(lambda: ops.embed_stream(x0, ids, table, 45.0, raw, wn, 0.0, 1e-6, hout))
+        rows.append(_row("embed_stream (scaled rows, raw rows, first norm)", phase, t, T * width * (2 + 4 + 2 + 2), 4.0 * T * width,
+                         VALU_F32))
+        split = torch.empty(T, 2 * width, dtype=bf, device=dev)
+        t = _time(lambda: ops.stream_split(split, stream, a, None, c32))
+        rows.append(_row("stream_split (two addends, one fp32)", phase, t, T * width * (4 + 4 + 2 + 4 + 4), 5.0 * T * width, VALU_F32))
+        t = _time(lambda: ops.stream_add_norm(stream, wn, 0.0, 1e-6, hout, a, None, c32))
+        rows.append(_row("stream_add_norm as Lapilorn runs it (two addends, one fp32)", phase, t, T * width * (4 + 4 + 2 + 4 + 2), 6.0 * T * width,
+                         VALU_F32, like="embed_stream, stream_split"))
+        w_loop = torch.randn(width, 2 * width, device=dev).to(bf) * 0.02
+        t = _time(lambda: torch.mm(split, w_loop.t(), out_dtype=torch.float32))
+        rows.append(_row("pass input: library GEMM of the split stream, fp32 out", phase, t,
+                         T * width * (4 + 4) + 4 * width * width, 4.0 * T * width * width, MFMA_BF16))
+        t = _time(lambda: torch.mm(split, w_loop.t()))
+        rows.append(_row("the same GEMM with bf16 out", phase, t, T * width * (4 + 2) + 4 * width * width,
+                         4.0 * T * width * width, MFMA_BF16, like="pass input"))
+        # ---------------------------------------------------------------- feed-forward
+        up = torch.randn(T, ff + 3072, device=dev).to(bf)
+        hidden, up_cols = both[:, :ff], up[:, :ff]
+        t = _time(lambda: ops.relu2(hidden, up_cols))
+        rows.append(_row("relu2 (column range into column range)", phase, t, T * ff * 2 * 2, 2.0 * T * ff, VALU_F32))
+        gu, act = torch.randn(T, 2 * ff, device=dev).to(bf), torch.empty(T, ff, dtype=bf, device=dev)
+        t = _time(lambda: ops.clamped_glu(act, gu, 1.702, 7.0, 1.0))
+        rows.append(_row("Lapilorn clamped_glu", phase, t, T * ff * 3 * 2, 8.0 * T * ff, VALU_F32, like="relu2"))
+        x = torch.randn(T, width, device=dev).to(bf)
+        router, rb = (torch.randn(experts, width, device=dev) * width ** -0.5), torch.randn(experts, device=dev) * 0.1
+        r16, eo = router.to(bf), torch.empty(T, width, device=dev)
+
+        def route():
+            return ops.group_router(torch.addmm(rb, x, r16.t(), out_dtype=torch.float32), None, top, 1, 1, 1.0,
+                                    ops.ROUTER_SOFTMAX_CHOSEN, clear=eo)
+        t = _time(route)
+        rows.append(_row("router: bf16 operands, fp32 products + choice, clears the sum", phase, t,
+                         T * width * (2 + 4) + experts * width * 2 + T * top * 8, 2.0 * T * experts * width, VALU_F32))
+
+        def route_bogetar():
+            torch.zeros(T, width, device=dev)
+            return ops.group_router(torch.matmul(x.float(), router.t()), None, top, 1, 1, 1.0, True, True, False)
+        t = _time(route_bogetar)
+        rows.append(_row("Bogetar router: fp32 copy + GEMM + choice, sum cleared apart", phase, t,
+                         T * width * (2 + 4) + experts * width * 4 + T * top * 8, 2.0 * T * experts * width, VALU_F32, like="router"))
+        chosen, weights = route()
+        order, start = ops.group_pairs(chosen, experts)
+        up_glu = (torch.randn(experts, 32 * (-(-expert_ff // 16)), width, device=dev) * 0.02).to(bf)
+        wd = (torch.randn(experts, width, expert_ff, device=dev) * 0.02).to(bf)
+        active = min(experts, T * top)
+        ebytes = active * 3 * expert_ff * width * 2 + T * width * (2 + 4) + T * top * expert_ff * 2 * 2
+        for name, glu, like in (("expert_ffn (silu gate)", (1.0, float("inf"), 0.0), ""),
+                                ("Bogetar expert_ffn (gated hidden layer with limits)", (1.702, 7.0, 1.0), "expert_ffn (silu gate)")):
+            t = _time(lambda: ops.expert_ffn(eo, x, up_glu, wd, order, start, top, 1.0, pair_weight=weights, glu=glu))
+            rows.append(_row(name, phase, t, ebytes, 6.0 * T * top * expert_ff * width, MFMA_BF16, like=like))
+    return rows
+
+
+# the existing families that a stack is measured beside
+_BESIDE = {"dovisun": ("lalasun", "bogetar", "llama")}
+
+
 def run(sizes=("2k",), with_kernels: bool = True, family: str = "nepevik") -> dict:
     result = {"family": family, "engine": {}, "kernels": {}}
     for size in sizes:
         pair = {}
-        for name in (family, "llama"):
+        for name in (family, *_BESIDE.get(family, ("llama",))):
             pair[name] = {k: round(v, 2) for k, v in engine_throughput(f"{name}-{size}").items()}
         result["engine"][size] = pair
     if with_kernels:
         table = {"nepevik": kernel_table, "lapilorn": kernel_table_lapilorn, "lalasun": kernel_table_lalasun,
-                 "bogetar": kernel_table_bogetar}[family]
+                 "bogetar": kernel_table_bogetar, "dovisun": kernel_table_dovisun}[family]
         result["kernels"]["2k"] = table()
     return result

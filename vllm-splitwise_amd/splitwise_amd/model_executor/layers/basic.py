@@ -343,21 +343,22 @@ class LoopInput(nn.Module):
         self.embed_weight.data.copy_(weight[:, w:])
 
     def start(self, rows: torch.Tensor) -> torch.Tensor:
-        """rows: the step's embedding rows, unscaled, in the activation dtype.  -> fp32 [rows, width]."""
+        """rows: the step's embedding rows, unscaled, in the activation dtype.  -> W_0 x_0, fp32 [rows, width]."""
         if rows.dtype == torch.float32:
-            return torch.mm(rows, self.embed_weight.data.t())
-        return torch.mm(rows, self.embed_weight.data.t(), out_dtype=torch.float32)
+            return torch.mm(rows, self.embed_weight.data.t()).mul_(self.scale)
+        return torch.mm(rows, self.embed_weight.data.t(), out_dtype=torch.float32).mul_(self.scale)
 
-    def forward(self, stream: torch.Tensor, from_embedding: torch.Tensor, a: Optional[torch.Tensor] = None,
-                b: Optional[torch.Tensor] = None, c: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """stream += a + b + c in place (the outputs of the layer before), then -> the new stream of the pass."""
+    def forward(self, stream: torch.Tensor, a: Optional[torch.Tensor] = None, b: Optional[torch.Tensor] = None,
+                c: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """stream += a + b + c in place (the outputs of the layer before), then -> W_x stream, fp32.  What ``start`` gave is
+        still to be added: the norm kernel of the pass's first layer takes it as an addend."""
         if self.dtype == torch.float32:
             if a is not None or b is not None or c is not None:
                 _C.mixer_ops.stream_add_norm(stream, None, 0.0, 0.0, None, a, b, c)
-            return torch.addmm(from_embedding, stream, self.stream_weight.data.t(), beta=self.scale)
+            return torch.mm(stream, self.stream_weight.data.t())
         split = torch.empty(stream.shape[0], 2 * self.width, dtype=self.dtype, device=stream.device)
         _C.mixer_ops.stream_split(split, stream, a, b, c)
-        return torch.addmm(from_embedding, split, self.stream_weight.data.t(), beta=self.scale, out_dtype=torch.float32)
+        return torch.mm(split, self.stream_weight.data.t(), out_dtype=torch.float32)
 
 
 class ClampedGLU(nn.Module):

@@ -162,7 +162,7 @@ class DovisunForCausalLM(nn.Module):
             raise NotImplementedError("Dovisun checkpoints are dense: no quantised linear method")
         self.config, self.dtype = cfg, dtype
         width, eps = cfg["width"], cfg["norm"]["eps"]
-        self.embed_scale = float(cfg["embedding"]["scale"])
+        self.embed_scale = float((cfg.get("embedding") or {}).get("scale", 1.0))
         self.runs = layer_runs(cfg)
         self.embed_tokens = VocabParallelEmbedding(cfg["vocab"], width, dtype)
         self.layers = nn.ModuleList([DovisunLayer(cfg, i, dtype, None) for i in range(len(cfg["layers"]))])
@@ -219,17 +219,17 @@ class DovisunForCausalLM(nn.Module):
                                       first.offset, first.variance_epsilon, h)
         from_embedding = loop.start(rows) if loop is not None else None
         if h is None:
-            x = loop(x, from_embedding)
-            h = first(x, self.dtype)
+            x = loop(x)
+            h = first.add_norm(x, self.dtype, None, None, from_embedding)
         for r, (i, _) in enumerate(self.runs):
             a, c = self.layers[i](h, positions, kv_caches[r], input_metadata)
             nxt = self._norm_of_run(r + 1)
             if r + 1 < n and self.runs[r + 1][1]:              # the next run begins a pass
-                x_new = loop(x, from_embedding, a, None, c)    # x += a + c;  x_new = the pass's input
+                x_new = loop(x, a, None, c)                    # x += a + c;  x_new = W_x x
                 if self.keep_residuals is not None:
                     self.keep_residuals.append(x.clone())
                 x = x_new
-                h = nxt(x, self.dtype)
+                h = nxt.add_norm(x, self.dtype, None, None, from_embedding)      # the pass's input and its norm
                 continue
             h = nxt.add_norm(x, self.dtype, a, None, c)        # x += a + c;  h = the next norm of x
             if self.keep_residuals is not None:
