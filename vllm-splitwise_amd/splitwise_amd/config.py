@@ -157,10 +157,9 @@ _BOGETAR_PRESETS = {
 
 def _dovisun_preset(width: int, repeats: int, heads: int, kv_heads: int, ff: int, experts: int, top: int,
                     expert_ff: int) -> dict:
-    """A Dovisun stack of layer sizes that resemble a served model's, ten layer runs per repeat of its one loop: a
-    latent-attention layer (a 384-wide query latent, a 192-wide key latent plus 64 rotated coordinates per token), a
-    block of two attention layers and a latent-attention layer that runs twice, and three layers behind it; dense
-    feed-forwards and routed experts in turn."""
+    """A Dovisun stack of layer sizes that resemble a served model's: a latent-attention layer (a 384-wide query latent, a
+    192-wide key latent plus 64 rotated coordinates per token), a block of two attention layers and a latent-attention
+    layer that runs ``repeats`` times, and three layers behind it; dense feed-forwards and routed experts in turn."""
     d = width // heads
     latent = {"heads": heads, "dim": d // 2, "rot_dim": 64, "vdim": d, "kv_rank": 192, "q_rank": 384,
               "scale": (d // 2 + 64) ** -0.5,
