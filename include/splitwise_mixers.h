@@ -11,8 +11,8 @@
  * step of layers that read a mix of all earlier layers' outputs; norms in groups of channels around every
  * sublayer, a causal convolution added to a sublayer's input, the delta rule with one decay per head, attention
  * with sigmoid weights and a softmax router; latent attention with a query latent, and the stream of decoders that run a
- * block of layers several times.  A library of its own so that a model that needs only these compiles
- * only these.
+ * block of layers several times; a residual of several streams, attention with a learned sink, retention.  A library of its
+ * own so that a model that needs only these compiles only these.
  *
  * A step is a RAGGED batch: the new tokens of all sequences back to back in one token dimension.
  *   q_start[B + 1]   first row of every sequence's tokens (int32, ascending, q_start[B] = rows)
@@ -37,7 +37,7 @@
 extern "C" {
 #endif
 
-#define SWM_ABI_VERSION 6
+#define SWM_ABI_VERSION 7
 int swm_abi_version(void);
 const char* swm_last_error(void);
 
@@ -258,7 +258,8 @@ int swm_latent_rope_cache(float* q_out, const void* q_latent, int64_t ql_row_str
                           const float* inv_freq, void* cache, const int64_t* slot_mapping, int64_t rows, int heads,
                           int rank, int rot, int act_dtype, void* stream);
 
-/* The per-head output norm with the gate's activation named: gate_silu != 0 multiplies by gate * sigmoid(gate). */
+/* The per-head output norm with the gate's activation named: gate_silu != 0 multiplies by gate * sigmoid(gate); weight NULL:
+ * all 1. */
 int swm_head_norm_gate_act(void* out, const float* o, const void* gate, int64_t gate_stride, const float* weight,
                            int weight_head_stride, float eps, int64_t rows, int heads, int vdim, int gate_silu,
                            int act_dtype, void* stream);
@@ -397,6 +398,66 @@ int swm_head_project(void* out, int out_dtype, int64_t out_row, int64_t out_head
                      const int64_t* positions, const float* inv_freq, int rot, int pair_halves, float amplitude,
                      const void* gate, int64_t gate_row, int gate_per_head, int64_t rows, int heads, int act_dtype,
                      void* stream);
+
+/* ---- a residual of several streams; attention with a learned sink; retention ---- */
+
+/* One step of a residual of num_streams fp32 streams (streams [rows, num_streams, width], 1..8 of them):
+ *   y = a + b + c   (each may be NULL; a, b act_dtype with row strides, c fp32 contiguous), or with a_norm and b_norm (fp32
+ *   [width]) y = blend * (N(a; a_norm) + N(b; b_norm)), N(u; w) = u / sqrt(mean(u^2) + eps) * w;
+ *   streams[t, j] <- sum_i mix[i, j] streams[t, i] + writes[j] * y[t], all j from the old streams (mix fp32 [num_streams,
+ *   num_streams], writes fp32 [num_streams]; both NULL: nothing is written);
+ *   out[t] = act_dtype(N(sum_j reads[j] streams[t, j]; weight))   (out NULL: none; reads fp32 [num_streams]).
+ * ids (int64 [rows], with table act_dtype [vocab, width]; NULL: none): every OLD stream of row t is table[ids[t]] and
+ * `streams` is only written (it may be NULL without a mix); an id beyond the table gives NaN. */
+int swm_hyper_step(float* streams, int num_streams, const int64_t* ids, const void* table, int64_t vocab, const float* mix,
+                   const float* writes, const void* a, int64_t a_stride, const void* b, int64_t b_stride, const float* c,
+                   const float* a_norm, const float* b_norm, float blend, const float* reads, const float* weight,
+                   float eps, void* out, int64_t rows, int width, int act_dtype, void* stream);
+
+/* in [rows, 2 * ff] = gate | up (row strides given): out = act(gate) * up, act = silu or the tanh form of gelu,
+ * 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))). */
+#define SWM_GATE_SILU 0
+#define SWM_GATE_GELU_TANH 1
+int swm_gated_act(void* out, int64_t out_stride, const void* in, int64_t in_stride, int64_t rows, int ff, int activation,
+                  int act_dtype, void* stream);
+
+/* The operands of one or two token mixers that share a projection output (all inputs: column ranges with row stride
+ * in_stride).  Rotation on the pairs (i, i + rot / 2) of every head by float(position) * inv_freq[i] (fp32 [rot / 2]), the
+ * coordinates from rot on pass.
+ * Attention side (q NULL: none): with q_norm and k_norm (fp32 [heads * dim], [kv_heads * dim]; NULL: none) q and k first
+ *   take ONE RMS norm each over the whole projection; q_out (fp32 [rows, heads * dim]) = turned q, key_cache[slot] = turned k,
+ *   value_cache[slot] = v (slot = slot_mapping[t], < 0: not cached).
+ * Linear side (lin_q NULL: none): lin_q_out, lin_k_out (fp32 [rows, lin_heads * lin_dim]) = turned q, turned k * lin_k_scale.
+ * Up to 512 rotated coordinates per head. */
+int swm_rope_operands(float* q_out, const void* q, const void* k, const void* v, const float* q_norm, const float* k_norm,
+                      float norm_eps, const float* inv_freq, int rot, int heads, int kv_heads, int dim, int vdim,
+                      void* key_cache, void* value_cache, const int64_t* slot_mapping, float* lin_q_out, float* lin_k_out,
+                      const void* lin_q, const void* lin_k, const float* lin_inv_freq, int lin_rot, int lin_heads,
+                      int lin_dim, float lin_k_scale, const int64_t* positions, int64_t in_stride, int64_t rows,
+                      int act_dtype, void* stream);
+
+/* swm_masked_attention whose extra softmax term is learned: the denominator of head h has one more term
+ * exp(sink_logit[h]) (fp32 [heads]; not scaled, no value). */
+int swm_sink_attention(void* out, int64_t out_stride, const float* q, const void* key_cache, const void* value_cache,
+                       const void* gate, int64_t gate_stride, const float* sink_logit, const int32_t* block_tables,
+                       int table_width, const int32_t* q_start, const int32_t* ctx_len, int64_t rows, int num_seqs,
+                       int max_query_len, int heads, int kv_heads, int dim, int vdim, int page_size, float scale,
+                       float softcap, int window, int chunk, int64_t k_stride, int64_t v_stride, float* workspace,
+                       int act_dtype, void* stream);
+
+/* The recurrence of swm_lightning on its operands as they are: q, k fp32 [rows, heads * dim] (row stride qk_stride), v
+ * act_dtype (row stride v_stride), no silu.  Workspace: swm_lightning_workspace_floats(). */
+int swm_retention(float* out, const float* q, const float* k, int64_t qk_stride, const void* v, int64_t v_stride,
+                  const float* decay, float* state, const int32_t* q_start, const int32_t* ctx_len,
+                  const int32_t* state_slot, int64_t rows, int num_seqs, int max_query_len, int heads, int dim, int vdim,
+                  float* workspace, int act_dtype, void* stream);
+
+/* swm_expert_up_as with a weight per (row, choice) pair on what the expert READS (fp32 [rows * top], NULL: all 1): the
+ * products are those of up[e] with pair_weight * x. */
+int swm_expert_up_weighted(void* hidden, const void* x, const void* up, const int32_t* order, const int32_t* expert_start,
+                           int num_experts, int64_t sorted_rows, int width, int ff, int top, int activation,
+                           float glu_alpha, float glu_limit, float glu_shift, const float* pair_weight, int act_dtype,
+                           void* stream);
 
 #ifdef __cplusplus
 }

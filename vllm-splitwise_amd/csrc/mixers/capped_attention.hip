@@ -1,7 +1,7 @@
 // Causal softmax attention of a ragged step over paged keys with grouped query heads, an optional soft cap on the
 // scores (cap * tanh(score / cap)), an optional mask (a sliding window, or chunks counted from position 0 inside which
-// a position sees the earlier ones), an optional extra term exp(0) in the softmax's denominator (a key of score 0
-// that carries no value) and an optional sigmoid gate on the output.  A cache slot's keys and values are addressed
+// a position sees the earlier ones), an optional extra term in the softmax's denominator (a key that carries no value, of
+// score 0 or of one learned score per query head) and an optional sigmoid gate on the output.  A cache slot's keys and values are addressed
 // by strides, so values may be a part of the key rows (attention over a latent shared by all heads).  Given a bias per
 // query head the same kernels run WITHOUT a softmax: a seen key weighs sigmoid(score + bias), nothing is normalised over
 // the keys, and parts are joined by plain addition.
@@ -118,7 +118,8 @@ __global__ __launch_bounds__(64 * max_waves_of(NB)) void capped_attention_kernel
     const void* __restrict__ value_cache, const void* __restrict__ gate, int64_t gate_stride,
     const int32_t* __restrict__ block_tables, int table_width, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_len, int num_seqs, int heads, int kv_heads, int dim, int vdim, int page_size,
-    float scale, float softcap, int window, int chunk, int sink, const float* __restrict__ score_bias, int64_t k_stride,
+    float scale, float softcap, int window, int chunk, int sink, const float* __restrict__ sink_logit,
+    const float* __restrict__ score_bias, int64_t k_stride,
     int64_t v_stride, int tpt, int split, int rows_used, int page_shift, float* __restrict__ partial,
     int64_t total_rows) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -318,7 +319,9 @@ __global__ __launch_bounds__(64 * max_waves_of(NB)) void capped_attention_kernel
       if (tt >= ntok) continue;
       float m_all = -INFINITY;
       for (int w = 0; w < nw; ++w) m_all = fmaxf(m_all, Ml[(w * kQT + r) * 2]);
-      if (sink) m_all = fmaxf(m_all, 0.0f);                  // one more term of score 0 that carries no value
+      // one more term that carries no value, of score 0 or of the head's learned score
+      const float sk = sink_logit != nullptr ? sink_logit[g * R + hh] : 0.0f;
+      if (sink) m_all = fmaxf(m_all, sk);
       if (partial != nullptr) {
         // this workgroup saw a part of the keys: its maximum, denominator and unnormalised sums go to the scratch that
         // the join kernel reads; the sink is the join's business
@@ -341,7 +344,7 @@ __global__ __launch_bounds__(64 * max_waves_of(NB)) void capped_attention_kernel
         po[pr * vdim + c] = num;
         continue;
       }
-      float num = 0.0f, den = sink ? expf(-m_all) : 0.0f;
+      float num = 0.0f, den = sink ? expf(sk - m_all) : 0.0f;
       for (int w = 0; w < nw; ++w) {
         const float f = expf(Ml[(w * kQT + r) * 2] - m_all);  // a wave that saw no key: exp(-inf) = 0
         den += f * Ml[(w * kQT + r) * 2 + 1];
@@ -357,9 +360,10 @@ __global__ __launch_bounds__(64 * max_waves_of(NB)) void capped_attention_kernel
   // ---- every wave for itself: turn O^T round through the wave's own LDS region (its queries are done with)
   __syncthreads();
   if (live) {
-    const float m_fin = sink ? fmaxf(m_run, 0.0f) : m_run;
+    const float sk = sink_logit != nullptr ? sink_logit[g * R + qi % R] : 0.0f;
+    const float m_fin = sink ? fmaxf(m_run, sk) : m_run;
     const float fin = sink ? expf(m_run - m_fin) : 1.0f;
-    const float inv = sig ? 1.0f : fin / (l_run * fin + (sink ? expf(-m_fin) : 0.0f));
+    const float inv = sig ? 1.0f : fin / (l_run * fin + (sink ? expf(sk - m_fin) : 0.0f));
 #pragma unroll
     for (int b = 0; b < NVB; ++b)
 #pragma unroll
@@ -389,7 +393,8 @@ __global__ __launch_bounds__(512) void capped_attention_rows_kernel(
     const void* __restrict__ value_cache, const void* __restrict__ gate, int64_t gate_stride,
     const int32_t* __restrict__ block_tables, int table_width, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_len, int heads, int kv_heads, int dim, int vdim, int page_size, int page_shift,
-    float scale, float softcap, int window, int chunk, int sink, const float* __restrict__ score_bias, int64_t k_stride,
+    float scale, float softcap, int window, int chunk, int sink, const float* __restrict__ sink_logit,
+    const float* __restrict__ score_bias, int64_t k_stride,
     int64_t v_stride) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int seq = blockIdx.x, g = blockIdx.y, R = heads / kv_heads;
@@ -502,8 +507,9 @@ __global__ __launch_bounds__(512) void capped_attention_rows_kernel(
     const int tt = r / R, hh = r % R;
     float m_all = -INFINITY;
     for (int w = 0; w < nw; ++w) m_all = fmaxf(m_all, Ml[(w * RQ + r) * 2]);
-    if (sink) m_all = fmaxf(m_all, 0.0f);
-    float num = 0.0f, den = sink ? expf(-m_all) : 0.0f;
+    const float sk = sink_logit != nullptr ? sink_logit[g * R + hh] : 0.0f;
+    if (sink) m_all = fmaxf(m_all, sk);
+    float num = 0.0f, den = sink ? expf(sk - m_all) : 0.0f;
     for (int w = 0; w < nw; ++w) {
       const float f = fast_expf_(Ml[(w * RQ + r) * 2] - m_all);      // a wave that saw no key: 0
       den += f * Ml[(w * RQ + r) * 2 + 1];
@@ -520,7 +526,7 @@ template <typename T, int RQ, int C, int LK>
 int launch_capped_rows(void* out, int64_t out_stride, const float* q, const void* key_cache, const void* value_cache, const void* gate,
                        int64_t gate_stride, const int32_t* block_tables, int table_width, const int32_t* q_start,
                        const int32_t* ctx_len, int num_seqs, int heads, int kv_heads, int dim, int vdim, int page_size,
-                       float scale, float softcap, int window, int chunk, int sink, const float* score_bias, int64_t k_stride,
+                       float scale, float softcap, int window, int chunk, int sink, const float* sink_logit, const float* score_bias, int64_t k_stride,
                        int64_t v_stride, hipStream_t stream) {
   constexpr bool half = sizeof(typename Conv<T>::store_t) == 2;
   constexpr int U = RQ * C <= 32 ? (half ? 4 : 2) : (half ? 2 : 1);
@@ -538,7 +544,7 @@ int launch_capped_rows(void* out, int64_t out_stride, const float* q, const void
   }
   hipLaunchKernelGGL(kernel, dim3((unsigned)num_seqs, (unsigned)kv_heads), dim3(64 * nw), lds_bytes, stream, out, out_stride, q,
                      key_cache, value_cache, gate, gate_stride, block_tables, table_width, q_start, ctx_len, heads,
-                     kv_heads, dim, vdim, page_size, page_shift, scale, softcap, window, chunk, sink, score_bias, k_stride,
+                     kv_heads, dim, vdim, page_size, page_shift, scale, softcap, window, chunk, sink, sink_logit, score_bias, k_stride,
                      v_stride);
   SW_CHECK_LAUNCH();
   return SW_OK;
@@ -550,7 +556,7 @@ bool try_capped_rows(int* status, int rows_used, void* out, int64_t out_stride, 
                      const void* value_cache, const void* gate, int64_t gate_stride, const int32_t* block_tables,
                      int table_width, const int32_t* q_start, const int32_t* ctx_len, int num_seqs, int heads,
                      int kv_heads, int dim, int vdim, int page_size, float scale, float softcap, int window, int chunk,
-                     int sink, const float* score_bias, int64_t k_stride, int64_t v_stride, hipStream_t stream) {
+                     int sink, const float* sink_logit, const float* score_bias, int64_t k_stride, int64_t v_stride, hipStream_t stream) {
   if (rows_used > 8) return false;
   auto pow2 = [](int x) { return x <= 4 ? 4 : x <= 8 ? 8 : x <= 16 ? 16 : x <= 32 ? 32 : 64; };
   const int most = std::max(dim, vdim);
@@ -566,7 +572,7 @@ bool try_capped_rows(int* status, int rows_used, void* out, int64_t out_stride, 
   if (rq == RQV && c == CV && lk == LKV) {                                                                              \
     *status = launch_capped_rows<T, RQV, CV, LKV>(out, out_stride, q, key_cache, value_cache, gate, gate_stride, block_tables,      \
                                                   table_width, q_start, ctx_len, num_seqs, heads, kv_heads, dim, vdim,  \
-                                                  page_size, scale, softcap, window, chunk, sink, score_bias, k_stride, \
+                                                  page_size, scale, softcap, window, chunk, sink, sink_logit, score_bias, k_stride, \
                                                   v_stride, stream);                                                              \
     return true;                                                                                                        \
   }
@@ -584,14 +590,15 @@ bool try_capped_rows(int* status, int rows_used, void* out, int64_t out_stride, 
 template <typename T>
 __global__ __launch_bounds__(256) void capped_attention_join_kernel(
     void* __restrict__ out, int64_t out_stride, const float* __restrict__ partial, const void* __restrict__ gate, int64_t gate_stride,
-    int64_t total_rows, int heads, int vdim, int parts, int sink, int sig) {
+    int64_t total_rows, int heads, int vdim, int parts, int sink, const float* __restrict__ sink_logit, int sig) {
   const int64_t rh = blockIdx.x;                             // row * heads + head
   const float* ml = partial;
   const float* po = partial + (int64_t)parts * total_rows * heads * 2;
   const int64_t part_stride = total_rows * heads;
-  float m_all = sink ? 0.0f : -INFINITY;
+  const float sk = sink_logit != nullptr ? sink_logit[rh % heads] : 0.0f;
+  float m_all = sink ? sk : -INFINITY;
   for (int z = 0; z < parts; ++z) m_all = fmaxf(m_all, ml[(z * part_stride + rh) * 2]);
-  float den = sink ? expf(-m_all) : 0.0f;
+  float den = sink ? expf(sk - m_all) : 0.0f;
   for (int z = 0; z < parts; ++z) {
     const float m = ml[(z * part_stride + rh) * 2];
     if (m != -INFINITY) den += expf(m - m_all) * ml[(z * part_stride + rh) * 2 + 1];
@@ -631,7 +638,7 @@ int launch_capped_attention(void* out, int64_t out_stride, const float* q, const
                             int64_t gate_stride, const int32_t* block_tables, int table_width, const int32_t* q_start,
                             const int32_t* ctx_len, int64_t rows, int num_seqs, int max_query_len, int heads,
                             int kv_heads, int dim, int vdim, int page_size, float scale, float softcap, int window,
-                            int chunk, int sink, const float* score_bias, int64_t k_stride, int64_t v_stride,
+                            int chunk, int sink, const float* sink_logit, const float* score_bias, int64_t k_stride, int64_t v_stride,
                             float* workspace, hipStream_t stream) {
   const int R = heads / kv_heads;
   const int tpt = kQT / R;
@@ -642,7 +649,7 @@ int launch_capped_attention(void* out, int64_t out_stride, const float* q, const
     int status = SW_OK;
     if (try_capped_rows<T>(&status, rows_used, out, out_stride, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width,
                            q_start, ctx_len, num_seqs, heads, kv_heads, dim, vdim, page_size, scale, softcap, window,
-                           chunk, sink, score_bias, k_stride, v_stride, stream))
+                           chunk, sink, sink_logit, score_bias, k_stride, v_stride, stream))
       return status;
   }
   auto lds_bytes = [&](int nw) {
@@ -673,12 +680,13 @@ int launch_capped_attention(void* out, int64_t out_stride, const float* q, const
   const dim3 grid((unsigned)(split ? tiles : (tiles + nw - 1) / nw), (unsigned)kv_heads, (unsigned)parts);
   hipLaunchKernelGGL(kernel, grid, dim3(64 * nw), lds_bytes(nw), stream, out, out_stride, q, key_cache, value_cache, gate,
                      gate_stride, block_tables, table_width, q_start, ctx_len, num_seqs, heads, kv_heads, dim, vdim,
-                     page_size, scale, softcap, window, chunk, sink, score_bias, k_stride, v_stride, tpt, split ? 1 : 0,
+                     page_size, scale, softcap, window, chunk, sink, sink_logit, score_bias, k_stride, v_stride, tpt, split ? 1 : 0,
                      rows_used, page_shift, parts > 1 ? workspace : (float*)nullptr, rows);
   SW_CHECK_LAUNCH();
   if (parts > 1) {
     hipLaunchKernelGGL(capped_attention_join_kernel<T>, dim3((unsigned)(rows * heads)), dim3(vdim <= 64 ? 64 : 128), 0,
-                       stream, out, out_stride, workspace, gate, gate_stride, rows, heads, vdim, parts, sink, score_bias != nullptr ? 1 : 0);
+                       stream, out, out_stride, workspace, gate, gate_stride, rows, heads, vdim, parts, sink,
+                       sink_logit, score_bias != nullptr ? 1 : 0);
     SW_CHECK_LAUNCH();
   }
   return SW_OK;
@@ -698,7 +706,7 @@ static int masked_attention_impl(void* out, int64_t out_stride, const float* q, 
                                  const void* gate, int64_t gate_stride, const int32_t* block_tables, int table_width,
                                  const int32_t* q_start, const int32_t* ctx_len, int64_t rows, int num_seqs,
                                  int max_query_len, int heads, int kv_heads, int dim, int vdim, int page_size,
-                                 float scale, float softcap, int window, int chunk, int sink, const float* score_bias,
+                                 float scale, float softcap, int window, int chunk, int sink, const float* sink_logit, const float* score_bias,
                                  int64_t k_stride, int64_t v_stride, float* workspace, int act_dtype, void* stream) {
   using namespace swm;
   if (rows == 0 || num_seqs == 0) return SW_OK;
@@ -723,7 +731,7 @@ static int masked_attention_impl(void* out, int64_t out_stride, const float* q, 
     SWM_DISPATCH_ACT(act_dtype, return (launch_capped_attention<T, N>(                                                  \
                                     out, out_stride, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width, \
                                     q_start, ctx_len, rows, num_seqs, max_query_len, heads, kv_heads, dim, vdim,        \
-                                    page_size, scale, softcap, window, chunk, sink, score_bias, k_stride, v_stride,     \
+                                    page_size, scale, softcap, window, chunk, sink, sink_logit, score_bias, k_stride, v_stride,     \
                                     workspace, s)););                                                                              \
     break;
   switch (nvb) {
@@ -756,7 +764,7 @@ extern "C" int swm_masked_attention(void* out, int64_t out_stride, const float* 
                                     int64_t k_stride, int64_t v_stride, float* workspace, int act_dtype, void* stream) {
   return masked_attention_impl(out, out_stride, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width,
                                q_start, ctx_len, rows, num_seqs, max_query_len, heads, kv_heads, dim, vdim, page_size, scale,
-                               softcap, window, chunk, sink, nullptr, k_stride, v_stride, workspace, act_dtype, stream);
+                               softcap, window, chunk, sink, nullptr, nullptr, k_stride, v_stride, workspace, act_dtype, stream);
 }
 
 extern "C" int swm_sigmoid_attention(void* out, const float* q, const void* key_cache, const void* value_cache,
@@ -771,7 +779,7 @@ extern "C" int swm_sigmoid_attention(void* out, const float* q, const void* key_
   }
   return masked_attention_impl(out, (int64_t)heads * vdim, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width, q_start,
                                ctx_len, rows, num_seqs, max_query_len, heads, kv_heads, dim, vdim, page_size, scale,
-                               0.0f, window, 0, 0, score_bias, (int64_t)kv_heads * dim, (int64_t)kv_heads * vdim,
+                               0.0f, window, 0, 0, nullptr, score_bias, (int64_t)kv_heads * dim, (int64_t)kv_heads * vdim,
                                workspace, act_dtype, stream);
 }
 
@@ -784,4 +792,20 @@ extern "C" int swm_capped_attention(void* out, const float* q, const void* key_c
                               ctx_len, rows, num_seqs, max_query_len, heads, kv_heads, dim, vdim, page_size, scale,
                               softcap, window, 0, 0, (int64_t)kv_heads * dim, (int64_t)kv_heads * vdim, nullptr, act_dtype,
                               stream);
+}
+
+extern "C" int swm_sink_attention(void* out, int64_t out_stride, const float* q, const void* key_cache, const void* value_cache,
+                                  const void* gate, int64_t gate_stride, const float* sink_logit,
+                                  const int32_t* block_tables, int table_width, const int32_t* q_start,
+                                  const int32_t* ctx_len, int64_t rows, int num_seqs, int max_query_len, int heads,
+                                  int kv_heads, int dim, int vdim, int page_size, float scale, float softcap, int window,
+                                  int chunk, int64_t k_stride, int64_t v_stride, float* workspace, int act_dtype,
+                                  void* stream) {
+  if (sink_logit == nullptr) {
+    sw::set_error("sink_attention: the score per head is missing");
+    return SW_ERR_INVALID;
+  }
+  return masked_attention_impl(out, out_stride, q, key_cache, value_cache, gate, gate_stride, block_tables, table_width,
+                               q_start, ctx_len, rows, num_seqs, max_query_len, heads, kv_heads, dim, vdim, page_size, scale,
+                               softcap, window, chunk, 1, sink_logit, nullptr, k_stride, v_stride, workspace, act_dtype, stream);
 }

@@ -56,7 +56,7 @@ template <typename T>
 __global__ __launch_bounds__(kFfnThreads) void expert_up_gelu_kernel(
     void* __restrict__ hidden, const void* __restrict__ x, const void* __restrict__ up,
     const int32_t* __restrict__ order, const int32_t* __restrict__ expert_start, int num_experts, int width, int ff,
-    int top, int activation, int up_rows, GluParams glu) {
+    int top, int activation, int up_rows, GluParams glu, const float* __restrict__ pair_weight) {
   __shared__ float As[TM][TK + 1];
   __shared__ float Bs[TN][TK + 1];
   int e, row0;
@@ -71,6 +71,11 @@ __global__ __launch_bounds__(kFfnThreads) void expert_up_gelu_kernel(
   for (int i = 0; i < 2; ++i) {
     const int r = 2 * ty + i;
     if (r >= rows) continue;
+    if (pair_weight != nullptr) {                            // the weight of the expert's INPUT, taken through the products
+      const float wt = pair_weight[order[row0 + r]];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[i][j] *= wt;
+    }
     if (activation == SWM_ACT_CLAMPED_GLU) {
       // columns tx + 16 j of the tile: j = 0, 2 are gate products, j = 1, 3 the up products of the same channels
 #pragma unroll
@@ -126,7 +131,7 @@ __global__ __launch_bounds__(kFfnThreads) void expert_down_kernel(
 __global__ __launch_bounds__(kFfnThreads) void expert_up_gelu_mfma_kernel(
     uint16_t* __restrict__ hidden, const uint16_t* __restrict__ x, const uint16_t* __restrict__ up,
     const int32_t* __restrict__ order, const int32_t* __restrict__ expert_start, int num_experts, int width, int ff,
-    int top, int activation, int up_rows, GluParams glu) {
+    int top, int activation, int up_rows, GluParams glu, const float* __restrict__ pair_weight) {
   __shared__ __attribute__((aligned(16))) uint16_t As[MM][MK + MPAD];
   __shared__ __attribute__((aligned(16))) uint16_t Bs[MN][MK + MPAD];
   int e, row0;
@@ -136,6 +141,14 @@ __global__ __launch_bounds__(kFfnThreads) void expert_up_gelu_mfma_kernel(
   f32x16 acc;
   tile_gemm_mfma<true>(acc, x, [&](int r) { return (int64_t)(order[row0 + r] / top) * width; }, rows, up, (int64_t)e * up_rows * width,
                  n0, up_rows, width, As, Bs);
+  if (pair_weight != nullptr) {                              // the weight of the expert's INPUT, taken through the products
+    const int r0 = (threadIdx.x >> 7) * 32 + 4 * ((threadIdx.x & 63) >> 5);
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const int r = r0 + 8 * (i / 4) + i % 4;                // this lane's rows, as for_each_acc counts them
+      if (r < rows) acc[i] *= pair_weight[order[row0 + r]];
+    }
+  }
   if (activation == SWM_ACT_CLAMPED_GLU) {
     // a lane's column c of the tile: c % 32 < 16 is the gate product of channel (n0 + c) / 32 * 16 + c % 16, and lane
     // + 16 holds the up product of the same channel and rows
@@ -197,6 +210,14 @@ int swm_expert_up(void* hidden, const void* x, const void* up, const int32_t* or
 int swm_expert_up_as(void* hidden, const void* x, const void* up, const int32_t* order, const int32_t* expert_start,
                      int num_experts, int64_t sorted_rows, int width, int ff, int top, int activation, float glu_alpha,
                      float glu_limit, float glu_shift, int act_dtype, void* stream) {
+  return swm_expert_up_weighted(hidden, x, up, order, expert_start, num_experts, sorted_rows, width, ff, top, activation,
+                                glu_alpha, glu_limit, glu_shift, nullptr, act_dtype, stream);
+}
+
+int swm_expert_up_weighted(void* hidden, const void* x, const void* up, const int32_t* order,
+                           const int32_t* expert_start, int num_experts, int64_t sorted_rows, int width, int ff, int top,
+                           int activation, float glu_alpha, float glu_limit, float glu_shift, const float* pair_weight,
+                           int act_dtype, void* stream) {
   using namespace swm;
   if (sorted_rows == 0) return SW_OK;
   const bool gated = activation == SWM_ACT_CLAMPED_GLU;
@@ -210,14 +231,14 @@ int swm_expert_up_as(void* hidden, const void* x, const void* up, const int32_t*
     const dim3 mgrid((unsigned)((sorted_rows + MM - 1) / MM + num_experts), (unsigned)((up_rows + MN - 1) / MN));
     hipLaunchKernelGGL(expert_up_gelu_mfma_kernel, mgrid, dim3(kFfnThreads), 0, static_cast<hipStream_t>(stream),
                        static_cast<uint16_t*>(hidden), static_cast<const uint16_t*>(x), static_cast<const uint16_t*>(up),
-                       order, expert_start, num_experts, width, ff, top, activation, up_rows, glu);
+                       order, expert_start, num_experts, width, ff, top, activation, up_rows, glu, pair_weight);
     SW_CHECK_LAUNCH();
     return SW_OK;
   }
   const dim3 grid((unsigned)((sorted_rows + TM - 1) / TM + num_experts), (unsigned)((up_rows + TN - 1) / TN));
   SWM_DISPATCH_ACT(act_dtype, hipLaunchKernelGGL(expert_up_gelu_kernel<T>, grid, dim3(kFfnThreads), 0,
                                                  static_cast<hipStream_t>(stream), hidden, x, up, order, expert_start,
-                                                 num_experts, width, ff, top, activation, up_rows, glu););
+                                                 num_experts, width, ff, top, activation, up_rows, glu, pair_weight););
   SW_CHECK_LAUNCH();
   return SW_OK;
 }

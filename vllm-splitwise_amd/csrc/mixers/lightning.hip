@@ -6,7 +6,8 @@
 //     O   = A V + diag(decay^(i + 1)) Q S                              (plus what the carried state holds)
 //     S  <- decay^n S + (K * decay^(n - 1 - j))^T V                    (n tokens in the chunk)
 // which is the recurrence itself with its sums reordered.  Powers of the decay come from a table built by
-// repeated multiplication, never from a quotient, so small decays do not overflow.
+// repeated multiplication, never from a quotient, so small decays do not overflow.  The same kernels run "retention":
+// the recurrence on fp32 queries and keys that the caller has rotated and scaled, and on the values as they are, no silu.
 //
 // One wave owns (sequence, head, 32 value channels) and keeps its slice of the state in registers across the
 // whole run (the waves of a workgroup share the chunk's queries and keys, staged once in LDS), in the matrix cores' accumulator layout (lane l: value channel l % 32; element r of block b:
@@ -25,10 +26,11 @@ constexpr int kSegment = 128;          // tokens per segment of a long run (a mu
 
 // NDB: 32-coordinate blocks of the key size.  A workgroup owns (sequence, head) and up to 8 blocks of 32 value
 // channels, one wave each; the chunk's silu(q) and silu(k) are staged once in LDS for all of them.
-template <typename T, int NDB>
+// TQ: type of queries and keys (row stride qk_stride), T: of the values (row stride v_stride); SILU: of all three.
+template <typename TQ, typename T, bool SILU, int NDB>
 __global__ __launch_bounds__(512) void lightning_kernel(
-    float* __restrict__ out, const void* __restrict__ q, const void* __restrict__ k, const void* __restrict__ v,
-    int64_t in_stride, const float* __restrict__ decay, float* __restrict__ state, const int32_t* __restrict__ q_start,
+    float* __restrict__ out, const void* __restrict__ q, const void* __restrict__ k, int64_t qk_stride,
+    const void* __restrict__ v, int64_t v_stride, const float* __restrict__ decay, float* __restrict__ state, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_len, const int32_t* __restrict__ state_slot, int num_seqs, int heads, int dim,
     int vdim, int mode, int seg_len, float* __restrict__ seg_state) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -80,26 +82,47 @@ __global__ __launch_bounds__(512) void lightning_kernel(
     }
 
   const int64_t qk_col = (int64_t)h * dim, v_col = (int64_t)h * vdim;
+  // fp32 operands in pieces of 4
+  const bool quads = sizeof(typename Conv<TQ>::store_t) == 4 && dim % 4 == 0 && qk_stride % 4 == 0 &&
+                     (reinterpret_cast<uintptr_t>(q) | reinterpret_cast<uintptr_t>(k)) % 16 == 0;
   for (int c0 = 0; c0 < n; c0 += kChunk) {
     const int cn = min(kChunk, n - c0);
-    const int64_t base = (int64_t)(row0 + c0) * in_stride;
+    const int64_t base = (int64_t)(row0 + c0) * qk_stride, v_base = (int64_t)(row0 + c0) * v_stride;
     __syncthreads();                                         // the last chunk's tiles have been read (and pw written)
-    for (int e = threadIdx.x; e < kChunk * NDB * 32; e += blockDim.x) {
-      const int r = e / (NDB * 32), c = e % (NDB * 32);
-      float qv = 0.0f, kv = 0.0f;
-      if (r < cn && c < dim) {
-        qv = fast_siluf_(ld<T>(q, base + r * in_stride + qk_col + c));
-        kv = fast_siluf_(ld<T>(k, base + r * in_stride + qk_col + c));
+    if (!SILU && quads) {
+      for (int e = threadIdx.x; e < kChunk * NDB * 8; e += blockDim.x) {
+        const int r = e / (NDB * 8), c = e % (NDB * 8) * 4;
+        float4 qv = make_float4(0.f, 0.f, 0.f, 0.f), kv = qv;
+        if (r < cn && c < dim) {
+          qv = *reinterpret_cast<const float4*>(static_cast<const float*>(q) + base + r * qk_stride + qk_col + c);
+          kv = *reinterpret_cast<const float4*>(static_cast<const float*>(k) + base + r * qk_stride + qk_col + c);
+        }
+        *reinterpret_cast<float4*>(Qs + r * DS + c) = qv;
+        *reinterpret_cast<float4*>(Ks + r * DS + c) = kv;
       }
-      Qs[r * DS + c] = qv;
-      Ks[r * DS + c] = kv;
+    } else {
+      for (int e = threadIdx.x; e < kChunk * NDB * 32; e += blockDim.x) {
+        const int r = e / (NDB * 32), c = e % (NDB * 32);
+        float qv = 0.0f, kv = 0.0f;
+        if (r < cn && c < dim) {
+          qv = ld<TQ>(q, base + r * qk_stride + qk_col + c);
+          kv = ld<TQ>(k, base + r * qk_stride + qk_col + c);
+          if (SILU) {
+            qv = fast_siluf_(qv);
+            kv = fast_siluf_(kv);
+          }
+        }
+        Qs[r * DS + c] = qv;
+        Ks[r * DS + c] = kv;
+      }
     }
     // ---- values of the chunk: channel vc of token (r, hl)
     float vt[16];
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int j = 8 * (r / 4) + 4 * hl + (r % 4);
-      vt[r] = (vc_ok && j < cn) ? fast_siluf_(ld<T>(v, base + j * in_stride + v_col + vc)) : 0.0f;
+      const float vv = (vc_ok && j < cn) ? ld<T>(v, v_base + j * v_stride + v_col + vc) : 0.0f;
+      vt[r] = SILU ? fast_siluf_(vv) : vv;                   // silu(0) = 0
     }
     __syncthreads();
     // ---- A^T = K Q^T (rows: keys, columns: queries); this lane: token li of the chunk as key and as query
@@ -220,15 +243,15 @@ __global__ __launch_bounds__(256) void lightning_scan_kernel(
   }
 }
 
-template <typename T, int NDB>
-int launch_lightning(float* out, const void* q, const void* k, const void* v, int64_t in_stride, const float* decay,
+template <typename TQ, typename T, bool SILU, int NDB>
+int launch_lightning(float* out, const void* q, const void* k, int64_t qk_stride, const void* v, int64_t v_stride, const float* decay,
                      float* state, const int32_t* q_start, const int32_t* ctx_len, const int32_t* state_slot,
                      int64_t rows, int num_seqs, int max_query_len, int heads, int dim, int vdim, float* seg_state,
                      hipStream_t stream) {
   const int vblocks = (vdim + 31) / 32;
   const int waves = std::min(vblocks, 8);
   const size_t lds_bytes = (size_t)(2 * kChunk * (NDB * 32 + 4) + kChunk + 2) * sizeof(float);
-  auto kernel = lightning_kernel<T, NDB>;
+  auto kernel = lightning_kernel<TQ, T, SILU, NDB>;
   static bool raised = false;                                // per instantiation
   if (lds_bytes > 64 * 1024 && !raised) {
     SW_CHECK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize,
@@ -238,22 +261,22 @@ int launch_lightning(float* out, const void* q, const void* k, const void* v, in
   const unsigned zgroups = (unsigned)((vblocks + waves - 1) / waves);
   if (seg_state == nullptr || max_query_len <= 2 * kSegment) {
     hipLaunchKernelGGL(kernel, dim3((unsigned)num_seqs, (unsigned)heads, zgroups), dim3(64 * waves), lds_bytes, stream,
-                       out, q, k, v, in_stride, decay, state, q_start, ctx_len, state_slot, num_seqs, heads, dim, vdim,
+                       out, q, k, qk_stride, v, v_stride, decay, state, q_start, ctx_len, state_slot, num_seqs, heads, dim, vdim,
                        kWhole, kSegment, seg_state);
     SW_CHECK_LAUNCH();
     return SW_OK;
   }
   const unsigned items = (unsigned)(rows / kSegment + num_seqs);
-  hipLaunchKernelGGL(kernel, dim3(items, (unsigned)heads, zgroups), dim3(64 * waves), lds_bytes, stream, out, q, k, v,
-                     in_stride, decay, state, q_start, ctx_len, state_slot, num_seqs, heads, dim, vdim, kLocal, kSegment,
+  hipLaunchKernelGGL(kernel, dim3(items, (unsigned)heads, zgroups), dim3(64 * waves), lds_bytes, stream, out, q, k,
+                     qk_stride, v, v_stride, decay, state, q_start, ctx_len, state_slot, num_seqs, heads, dim, vdim, kLocal, kSegment,
                      seg_state);
   SW_CHECK_LAUNCH();
   hipLaunchKernelGGL(lightning_scan_kernel, dim3((unsigned)num_seqs, (unsigned)heads, (unsigned)((dim * vdim + 255) / 256)),
                      dim3(256), 0, stream, seg_state, state, decay, q_start, ctx_len, state_slot, heads, dim, vdim,
                      kSegment);
   SW_CHECK_LAUNCH();
-  hipLaunchKernelGGL(kernel, dim3(items, (unsigned)heads, zgroups), dim3(64 * waves), lds_bytes, stream, out, q, k, v,
-                     in_stride, decay, state, q_start, ctx_len, state_slot, num_seqs, heads, dim, vdim, kFinal, kSegment,
+  hipLaunchKernelGGL(kernel, dim3(items, (unsigned)heads, zgroups), dim3(64 * waves), lds_bytes, stream, out, q, k,
+                     qk_stride, v, v_stride, decay, state, q_start, ctx_len, state_slot, num_seqs, heads, dim, vdim, kFinal, kSegment,
                      seg_state);
   SW_CHECK_LAUNCH();
   return SW_OK;
@@ -277,11 +300,12 @@ extern "C" int swm_lightning(float* out, const void* q, const void* k, const voi
   SW_CHECK_ARG(heads > 0 && heads < 65536 && dim > 0 && dim <= 256 && vdim > 0 && (vdim + 255) / 256 < 65536,
                "lightning: %d heads, key size %d (at most 256), value size %d", heads, dim, vdim);
   hipStream_t s = static_cast<hipStream_t>(stream);
-#define SWM_LIGHTNING_CASE(N)                                                                                       \
-  case N:                                                                                                           \
-    SWM_DISPATCH_ACT(act_dtype, return (launch_lightning<T, N>(out, q, k, v, in_stride, decay, state, q_start,      \
-                                                               ctx_len, state_slot, rows, num_seqs, max_query_len,  \
-                                                               heads, dim, vdim, workspace, s)););                  \
+#define SWM_LIGHTNING_CASE(N)                                                                                             \
+  case N:                                                                                                                 \
+    SWM_DISPATCH_ACT(act_dtype, return (launch_lightning<T, T, true, N>(out, q, k, in_stride, v, in_stride, decay, state, \
+                                                                        q_start, ctx_len, state_slot, rows, num_seqs,     \
+                                                                        max_query_len, heads, dim, vdim, workspace,       \
+                                                                        s)););                                            \
     break;
   switch ((dim + 31) / 32) {
     SWM_LIGHTNING_CASE(1)
@@ -294,5 +318,36 @@ extern "C" int swm_lightning(float* out, const void* q, const void* k, const voi
     SWM_LIGHTNING_CASE(8)
   }
 #undef SWM_LIGHTNING_CASE
+  return SW_OK;
+}
+
+extern "C" int swm_retention(float* out, const float* q, const float* k, int64_t qk_stride, const void* v, int64_t v_stride,
+                             const float* decay, float* state, const int32_t* q_start, const int32_t* ctx_len,
+                             const int32_t* state_slot, int64_t rows, int num_seqs, int max_query_len, int heads, int dim,
+                             int vdim, float* workspace, int act_dtype, void* stream) {
+  using namespace swm;
+  if (rows == 0 || num_seqs == 0) return SW_OK;
+  SW_CHECK_ARG(act_ok(act_dtype), "retention: unsupported dtype %d", act_dtype);
+  SW_CHECK_ARG(heads > 0 && heads < 65536 && dim > 0 && dim <= 256 && vdim > 0 && (vdim + 255) / 256 < 65536,
+               "retention: %d heads, key size %d (at most 256), value size %d", heads, dim, vdim);
+  hipStream_t s = static_cast<hipStream_t>(stream);
+#define SWM_RETENTION_CASE(N)                                                                                          \
+  case N:                                                                                                              \
+    SWM_DISPATCH_ACT(act_dtype, return (launch_lightning<float, T, false, N>(out, q, k, qk_stride, v, v_stride, decay, \
+                                                                             state, q_start, ctx_len, state_slot,      \
+                                                                             rows, num_seqs, max_query_len, heads,     \
+                                                                             dim, vdim, workspace, s)););              \
+    break;
+  switch ((dim + 31) / 32) {
+    SWM_RETENTION_CASE(1)
+    SWM_RETENTION_CASE(2)
+    SWM_RETENTION_CASE(3)
+    SWM_RETENTION_CASE(4)
+    SWM_RETENTION_CASE(5)
+    SWM_RETENTION_CASE(6)
+    SWM_RETENTION_CASE(7)
+    SWM_RETENTION_CASE(8)
+  }
+#undef SWM_RETENTION_CASE
   return SW_OK;
 }

@@ -113,7 +113,7 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(
   for (int c = lane; c < vdim; c += 64) {
     const float gv = ld<T>(gate, t * gate_stride + h * vdim + c);
     const float g = gate_silu ? gv * sigmoidf_(gv) : sigmoidf_(gv);
-    st<T>(out, (t * heads + h) * (int64_t)vdim + c, src[c] * f * weight[h * weight_head_stride + c] * g);
+    st<T>(out, (t * heads + h) * (int64_t)vdim + c, src[c] * f * (weight != nullptr ? weight[h * weight_head_stride + c] : 1.0f) * g);
   }
 }
 

@@ -18,7 +18,7 @@ import torch
 
 _PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 _LIB_PATH = os.path.join(_PKG_DIR, "libsplitwise_mixers.so")
-ABI_VERSION = 6
+ABI_VERSION = 7
 
 SW_F32, SW_BF16 = 0, 2
 _ACT = {torch.float32: SW_F32, torch.bfloat16: SW_BF16}
@@ -70,10 +70,19 @@ _SIGNATURES = {
     "swm_latent_down": [_p, _p, _i, _p, _p, _i, _p, _l, _f, _p, _p, _i, _i, _f, _p, _p, _l, _i, _p],
     "swm_head_project": [_p, _i, _l, _l, _p, _l, _l, _p, _i, _i, _p, _l, _l, _p, _p, _i, _i, _f, _p, _l, _i, _l, _i, _i,
                          _p],
+    "swm_hyper_step": [_p, _i, _p, _p, _l, _p, _p, _p, _l, _p, _l, _p, _p, _p, _f, _p, _p, _f, _p, _l, _i, _i, _p],
+    "swm_gated_act": [_p, _l, _p, _l, _l, _i, _i, _i, _p],
+    "swm_rope_operands": [_p, _p, _p, _p, _p, _p, _f, _p, _i, _i, _i, _i, _i, _p, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _f,
+                          _p, _l, _l, _i, _p],
+    "swm_sink_attention": [_p, _l, _p, _p, _p, _p, _l, _p, _p, _i, _p, _p, _l, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i,
+                           _l, _l, _p, _i, _p],
+    "swm_retention": [_p, _p, _p, _l, _p, _l, _p, _p, _p, _p, _p, _l, _i, _i, _i, _i, _i, _p, _i, _p],
+    "swm_expert_up_weighted": [_p, _p, _p, _p, _p, _i, _l, _i, _i, _i, _i, _f, _f, _f, _p, _i, _p],
     "swm_expert_up_as": [_p, _p, _p, _p, _p, _i, _l, _i, _i, _i, _i, _f, _f, _f, _i, _p],
 }
 ACT_GELU, ACT_RELU2, ACT_NONE, ACT_CLAMPED_GLU = 0, 1, 2, 3
 ROUTER_SOFTMAX, ROUTER_SOFTMAX_CHOSEN = 1, 2
+GATE_SILU, GATE_GELU_TANH = 0, 1
 
 _lib = None
 
@@ -415,33 +424,37 @@ def general_delta(out: torch.Tensor, r: torch.Tensor, k: torch.Tensor, v: torch.
             _stream(r)))
 
 
-def head_norm_gate(out: torch.Tensor, o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, per_head_weight: bool,
-                   eps: float, heads: int, vdim: int, gate_silu: bool = False) -> None:
-    """``per_head_weight``: weight is [heads * vdim]; otherwise [vdim], shared by the heads.  ``gate_silu``: the
-    normed output is multiplied by gate * sigmoid(gate) instead of sigmoid(gate)."""
+def head_norm_gate(out: torch.Tensor, o: torch.Tensor, gate: torch.Tensor, weight: Optional[torch.Tensor],
+                   per_head_weight: bool, eps: float, heads: int, vdim: int, gate_silu: bool = False) -> None:
+    """``per_head_weight``: weight is [heads * vdim]; otherwise [vdim], shared by the heads (None: no weight).
+    ``gate_silu``: the normed output is multiplied by gate * sigmoid(gate) instead of sigmoid(gate)."""
     _dev(out, o, gate, weight)
     _f32c(o, "o")
-    _f32c(weight, "weight")
+    if weight is not None:
+        _f32c(weight, "weight")
     rows = o.shape[0]
     _need(o.shape == (rows, heads * vdim) and gate.shape == o.shape and out.shape == o.shape and out.is_contiguous()
-          and out.dtype == gate.dtype and weight.numel() == (heads * vdim if per_head_weight else vdim),
+          and out.dtype == gate.dtype
+          and (weight is None or weight.numel() == (heads * vdim if per_head_weight else vdim)),
           "head_norm_gate: shapes")
     with _on_device_of(o):
         _check(load_library().swm_head_norm_gate_act(out.data_ptr(), o.data_ptr(), gate.data_ptr(),
-                                                     _rows(gate, "gate"), weight.data_ptr(),
+                                                     _rows(gate, "gate"), _opt_ptr(weight),
                                                      vdim if per_head_weight else 0, eps, rows, heads, vdim,
                                                      1 if gate_silu else 0, _act(out), _stream(o)))
 
 
 def expert_ffn(out: torch.Tensor, x: torch.Tensor, up: torch.Tensor, down: torch.Tensor, order: torch.Tensor,
                expert_start: torch.Tensor, top: int, weight: float, activation: int = ACT_GELU,
-               pair_weight: Optional[torch.Tensor] = None, glu: Optional[tuple] = None) -> None:
+               pair_weight: Optional[torch.Tensor] = None, glu: Optional[tuple] = None,
+               weigh_input: bool = False) -> None:
     """out (fp32 [rows, width], zeroed by the caller) += weight * sum over each row's experts of
     pair_weight[row, choice] * down[e] act(up[e] x[row]); ``order`` / ``expert_start``: the (row, choice) pairs
     sorted by expert and every expert's first sorted pair; ``activation``: ACT_GELU (exact gelu) or ACT_RELU2;
     ``pair_weight`` fp32 [rows, top] (None: all 1).  ``glu`` = (alpha, limit, shift): a gated hidden layer,
     g sigmoid(alpha g) (u + shift) with g = min(gate x, limit), u = clamp(up x, -limit, limit), worked out in the
-    up-projection's epilogue -- ``up`` then holds gate and up rows in runs of 16 (``glu_rows``)."""
+    up-projection's epilogue -- ``up`` then holds gate and up rows in runs of 16 (``glu_rows``).  ``weigh_input``: the pair's
+    weight multiplies what the expert reads instead of what it returns."""
     _dev(out, x, up, down, order, expert_start, pair_weight)
     _f32c(out, "out")
     rows, width = x.shape
@@ -465,12 +478,12 @@ def expert_ffn(out: torch.Tensor, x: torch.Tensor, up: torch.Tensor, down: torch
     hidden = torch.empty(pairs, ff, dtype=x.dtype, device=x.device)
     with _on_device_of(x):
         lib = load_library()
-        _check(lib.swm_expert_up_as(hidden.data_ptr(), x.data_ptr(), up.data_ptr(), order.data_ptr(),
-                                    expert_start.data_ptr(), experts, pairs, width, ff, top, activation, alpha, limit,
-                                    shift, _act(x), _stream(x)))
+        _check(lib.swm_expert_up_weighted(hidden.data_ptr(), x.data_ptr(), up.data_ptr(), order.data_ptr(),
+                                          expert_start.data_ptr(), experts, pairs, width, ff, top, activation, alpha, limit,
+                                          shift, _opt_ptr(pair_weight) if weigh_input else None, _act(x), _stream(x)))
         _check(lib.swm_expert_down_weighted(out.data_ptr(), hidden.data_ptr(), down.data_ptr(), order.data_ptr(),
                                             expert_start.data_ptr(), experts, pairs, width, ff, top, weight,
-                                            None if pair_weight is None else pair_weight.data_ptr(), _act(x),
+                                            None if weigh_input else _opt_ptr(pair_weight), _act(x),
                                             _stream(x)))
 
 
@@ -664,18 +677,22 @@ def group_pairs(chosen: torch.Tensor, experts: int):
 
 def capped_attention(out: torch.Tensor, q: torch.Tensor, key_cache: torch.Tensor, value_cache: Optional[torch.Tensor],
                      gate: Optional[torch.Tensor], batch, heads: int, kv_heads: int, dim: int, vdim: int, scale: float,
-                     softcap: float = 0.0, window: int = 0, chunk: int = 0, sink: bool = False,
+                     softcap: float = 0.0, window: int = 0, chunk: int = 0, sink: Union[bool, torch.Tensor] = False,
                      score_bias: Optional[torch.Tensor] = None) -> None:
     """out [rows, heads * vdim] (cache dtype; a column range of wider rows is fine, but not with ``score_bias``); q fp32
     [rows, heads * dim]; caches [pages, page, kv_heads * size]; gate (None: no gate): a 2-D view [rows, heads * vdim] in the cache dtype.  ``window`` / ``chunk``: the mask (a
-    sliding window, or chunks counted from position 0; neither: plain causal); ``sink``: one more term exp(0) in the
-    softmax's denominator.  ``value_cache`` None: a token's values are the first kv_heads * vdim elements of its
+    sliding window, or chunks counted from position 0; neither: plain causal); ``sink``: one more term in the softmax's
+    denominator, exp(0), or exp(sink[head]) when it is a tensor (fp32 [heads]).  ``value_cache`` None: a token's values are the first kv_heads * vdim elements of its
     key row (attention over a shared latent).  ``score_bias`` (fp32 [heads]): no softmax -- a seen key weighs
     sigmoid(score + score_bias[head]) and the weights are not normalised (window mask only)."""
-    _dev(out, q, key_cache, value_cache, gate, score_bias)
+    learned = sink if isinstance(sink, torch.Tensor) else None
+    _dev(out, q, key_cache, value_cache, gate, score_bias, learned)
+    if learned is not None:
+        _f32c(learned, "sink")
+        _need(learned.numel() == heads and score_bias is None, "capped_attention: one sink per query head, under a softmax")
     if score_bias is not None:
         _f32c(score_bias, "score_bias")
-        _need(score_bias.numel() == heads and not softcap and not chunk and not sink,
+        _need(score_bias.numel() == heads and not softcap and not chunk and sink is False,
               "capped_attention: sigmoid weights take a bias per head and no cap, chunks or sink")
     _f32c(q, "q")
     rows = q.shape[0]
@@ -716,6 +733,14 @@ def capped_attention(out: torch.Tensor, q: torch.Tensor, key_cache: torch.Tensor
                 0 if gate is None else _rows(gate, "gate"), score_bias.data_ptr(), tables.data_ptr(), tables.shape[1],
                 batch.q_start.data_ptr(), batch.ctx_len.data_ptr(), rows, n, longest, heads, kv_heads, dim, vdim,
                 key_cache.shape[1], scale, int(window), _opt_ptr(work), _act(out), _stream(q)))
+            return
+        if learned is not None:
+            _check(lib.swm_sink_attention(
+                out.data_ptr(), out_stride, q.data_ptr(), key_cache.data_ptr(), value_cache.data_ptr(), _opt_ptr(gate),
+                0 if gate is None else _rows(gate, "gate"), learned.data_ptr(), tables.data_ptr(), tables.shape[1],
+                batch.q_start.data_ptr(), batch.ctx_len.data_ptr(), rows, n, longest, heads, kv_heads, dim, vdim,
+                key_cache.shape[1], scale, softcap, int(window), int(chunk), k_stride, v_stride, _opt_ptr(work), _act(out),
+                _stream(q)))
             return
         _check(lib.swm_masked_attention(
             out.data_ptr(), out_stride, q.data_ptr(), key_cache.data_ptr(), value_cache.data_ptr(), _opt_ptr(gate),
@@ -1015,6 +1040,147 @@ def lightning(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tens
                                  _act(q), _stream(q)))
 
 
+def retention(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor,
+              state: torch.Tensor, batch, heads: int, dim: int, vdim: int) -> None:
+    """S <- decay[h] S + k v^T;  o = S^T q.  out fp32 [rows, heads * vdim]; q, k fp32 [rows, heads * dim] (the caller's
+    rotation and scale are in them); v: a 2-D view in an activation dtype; decay fp32 [heads]; state fp32 [slots, heads,
+    dim, vdim]."""
+    _dev(out, q, k, v, decay, state)
+    for t, what in ((out, "out"), (q, "q"), (k, "k"), (decay, "decay"), (state, "state")):
+        _f32c(t, what)
+    rows = q.shape[0]
+    n = _ragged_ok(batch, rows)
+    _need(q.shape == (rows, heads * dim) and k.shape == q.shape and v.shape == (rows, heads * vdim)
+          and out.shape == (rows, heads * vdim) and decay.numel() == heads and state.shape[1:] == (heads, dim, vdim)
+          and batch.max_state_slot < state.shape[0], "retention: shapes")
+    longest = int(getattr(batch, "max_query_len", 0) or 0)
+    with _on_device_of(q):
+        lib = load_library()
+        need = lib.swm_lightning_workspace_floats(rows, n, longest, heads, dim, vdim)
+        work = torch.empty(need, dtype=torch.float32, device=q.device) if need > 0 else None
+        _check(lib.swm_retention(out.data_ptr(), q.data_ptr(), k.data_ptr(), heads * dim, v.data_ptr(), _rows(v, "v"),
+                                 decay.data_ptr(), state.data_ptr(), batch.q_start.data_ptr(), batch.ctx_len.data_ptr(),
+                                 batch.state_slot.data_ptr(), rows, n, longest, heads, dim, vdim, _opt_ptr(work), _act(v),
+                                 _stream(q)))
+
+
+def hyper_step(streams: Optional[torch.Tensor], out: Optional[torch.Tensor], eps: float,
+               origin: Optional[tuple] = None, mix: Optional[torch.Tensor] = None, writes: Optional[torch.Tensor] = None,
+               a: Optional[torch.Tensor] = None, b: Optional[torch.Tensor] = None, c: Optional[torch.Tensor] = None,
+               norms: Optional[tuple] = None, blend: float = 1.0, reads: Optional[torch.Tensor] = None,
+               weight: Optional[torch.Tensor] = None) -> None:
+    """streams fp32 [rows, S, width], in place:  x_j <- sum_i mix[i, j] x_i + writes[j] * y, y = a + b + c (a, b: 2-D views in
+    the activation dtype, c fp32) or, with ``norms`` = (a's, b's norm weight), y = blend * (N(a) + N(b)); then out =
+    N(sum_j reads[j] x_j; weight).  ``origin`` = (ids int64 [rows], table [vocab, width]): the old streams of a row are all
+    table[ids[row]] (``streams`` is only written; None without a mix)."""
+    ids, table = origin if origin is not None else (None, None)
+    na, nb = norms if norms is not None else (None, None)
+    _dev(streams, out, ids, table, mix, writes, a, b, c, na, nb, reads, weight)
+    if streams is not None:
+        _f32c(streams, "streams")
+        _need(streams.dim() == 3, "hyper_step: streams must be [rows, S, width]")
+        rows, s, width = streams.shape
+    else:
+        _need(origin is not None and mix is None and out is not None and reads is not None, "hyper_step: no streams")
+        (rows, width), s = out.shape, reads.numel()
+    act = table if table is not None else out if out is not None else a if a is not None else b
+    if origin is not None:
+        _need(ids.dtype == torch.int64 and ids.is_contiguous() and ids.numel() == rows and table.dim() == 2
+              and table.is_contiguous() and table.shape[1] == width, "hyper_step: ids and table")
+    if mix is not None:
+        _f32c(mix, "mix")
+        _f32c(writes, "writes")
+        _need(mix.shape == (s, s) and writes.numel() == s and streams is not None, "hyper_step: mix and writes")
+        for t in (a, b):
+            _need(t is None or (t.shape == (rows, width) and (act is None or t.dtype == act.dtype)), "hyper_step: addend")
+        if c is not None:
+            _f32c(c, "c")
+            _need(c.shape == (rows, width), "hyper_step: fp32 addend")
+    else:
+        _need(a is None and b is None and c is None and norms is None, "hyper_step: an addend without a mix")
+    if norms is not None:
+        _f32c(na, "norm weight")
+        _f32c(nb, "norm weight")
+        _need(na.numel() == width and nb.numel() == width and a is not None and b is not None and c is None,
+              "hyper_step: normed outputs come in twos")
+    if out is not None:
+        _f32c(reads, "reads")
+        _f32c(weight, "weight")
+        _need(out.shape == (rows, width) and out.is_contiguous() and reads.numel() == s and weight.numel() == width
+              and out.dtype == act.dtype, "hyper_step: out")
+    dev = streams if streams is not None else out
+    with _on_device_of(dev):
+        _check(load_library().swm_hyper_step(
+            _opt_ptr(streams), s, _opt_ptr(ids), _opt_ptr(table), 0 if table is None else table.shape[0], _opt_ptr(mix),
+            _opt_ptr(writes), _opt_ptr(a), 0 if a is None else _rows(a, "a"), _opt_ptr(b), 0 if b is None else _rows(b, "b"),
+            _opt_ptr(c), _opt_ptr(na), _opt_ptr(nb), blend, _opt_ptr(reads), _opt_ptr(weight), eps, _opt_ptr(out), rows, width,
+            SW_F32 if act is None else _act(act), _stream(dev)))
+
+
+def gated_act(out: torch.Tensor, gate_up: torch.Tensor, activation: int = GATE_SILU) -> None:
+    """gate_up [rows, 2 * ff] = gate | up -> out [rows, ff] = act(gate) * up, act = GATE_SILU or GATE_GELU_TANH; both 2-D
+    views."""
+    _dev(out, gate_up)
+    rows, ff = out.shape
+    _need(gate_up.shape == (rows, 2 * ff) and gate_up.dtype == out.dtype, "gated_act: shapes")
+    with _on_device_of(out):
+        _check(load_library().swm_gated_act(out.data_ptr(), _rows(out, "out"), gate_up.data_ptr(), _rows(gate_up, "gate_up"),
+                                            rows, ff, activation, _act(out), _stream(out)))
+
+
+def rope_operands(positions: torch.Tensor, attention: Optional[tuple] = None, linear: Optional[tuple] = None,
+                  q_norm: Optional[torch.Tensor] = None, k_norm: Optional[torch.Tensor] = None, norm_eps: float = 0.0) -> None:
+    """The operands of one or two token mixers from column ranges of ONE projection output, rotated on the pairs
+    (i, i + rot / 2) by position * inv_freq[i].
+    ``attention`` = (q_out fp32, q, k, v, inv_freq, heads, kv_heads, dim, vdim, key_cache, value_cache, slot_mapping); with
+    ``q_norm`` / ``k_norm`` (fp32, one number per row of the projection) q and k first get one RMS norm over ALL heads.
+    ``linear`` = (q_out fp32, k_out fp32, q, k, inv_freq, heads, dim, k_scale)."""
+    args_a, args_l = [None] * 4 + [q_norm, k_norm, norm_eps, None, 0, 0, 0, 0, 0, None, None, None], [None] * 5 + [0, 0, 0, 0.0]
+    first = None
+    if attention is not None:
+        q_out, q, k, v, inv_freq, heads, kv_heads, dim, vdim, key_cache, value_cache, slot_mapping = attention
+        _dev(q_out, q, k, v, inv_freq, key_cache, value_cache, slot_mapping, q_norm, k_norm)
+        first, rows, stride = q, q.shape[0], _rows(q, "q")
+        _f32c(q_out, "q_out")
+        _f32c(inv_freq, "inv_freq")
+        _need(q.shape == (rows, heads * dim) and q_out.shape == q.shape and k.shape == (rows, kv_heads * dim)
+              and v.shape == (rows, kv_heads * vdim) and _rows(k, "k") == stride and _rows(v, "v") == stride
+              and k.dtype == q.dtype and v.dtype == q.dtype and 2 * inv_freq.numel() <= dim,
+              "rope_operands: q, k, v must share rows, stride and dtype")
+        _need(key_cache.dtype == q.dtype and value_cache.dtype == q.dtype and key_cache.is_contiguous()
+              and value_cache.is_contiguous() and key_cache.shape[-1] == kv_heads * dim
+              and value_cache.shape[-1] == kv_heads * vdim
+              and key_cache.shape[0] * key_cache.shape[1] == value_cache.shape[0] * value_cache.shape[1],
+              "rope_operands: cache shapes")
+        _slots_ok(slot_mapping, rows)
+        if q_norm is not None:
+            _f32c(q_norm, "q_norm")
+            _f32c(k_norm, "k_norm")
+            _need(q_norm.numel() == heads * dim and k_norm.numel() == kv_heads * dim, "rope_operands: norm weights")
+        args_a = [q_out.data_ptr(), q.data_ptr(), k.data_ptr(), v.data_ptr(), _opt_ptr(q_norm), _opt_ptr(k_norm), norm_eps,
+                  inv_freq.data_ptr(), 2 * inv_freq.numel(), heads, kv_heads, dim, vdim, key_cache.data_ptr(),
+                  value_cache.data_ptr(), slot_mapping.data_ptr()]
+    if linear is not None:
+        lq_out, lk_out, lq, lk, l_freq, l_heads, l_dim, k_scale = linear
+        _dev(lq_out, lk_out, lq, lk, l_freq)
+        for t, what in ((lq_out, "q_out"), (lk_out, "k_out"), (l_freq, "inv_freq")):
+            _f32c(t, what)
+        if first is None:
+            first, rows, stride = lq, lq.shape[0], _rows(lq, "q")
+        _need(lq.shape == (rows, l_heads * l_dim) and lk.shape == lq.shape and lq_out.shape == lq.shape
+              and lk_out.shape == lq.shape and _rows(lq, "q") == stride and _rows(lk, "k") == stride
+              and lq.dtype == first.dtype and lk.dtype == first.dtype and 2 * l_freq.numel() <= l_dim,
+              "rope_operands: the linear side's q and k must share rows, stride and dtype")
+        args_l = [lq_out.data_ptr(), lk_out.data_ptr(), lq.data_ptr(), lk.data_ptr(), l_freq.data_ptr(), 2 * l_freq.numel(),
+                  l_heads, l_dim, k_scale]
+    _need(first is not None, "rope_operands: nothing to do")
+    _need(positions.dtype == torch.int64 and positions.numel() == rows and positions.is_contiguous() and positions.is_cuda,
+          "rope_operands: positions must be int64 [rows]")
+    with _on_device_of(first):
+        _check(load_library().swm_rope_operands(*args_a, *args_l, positions.data_ptr(), stride, rows, _act(first),
+                                                _stream(first)))
+
+
 ops = SimpleNamespace(expert_ffn=expert_ffn, ACT_GELU=ACT_GELU, ACT_RELU2=ACT_RELU2,
     scalar_norm_add=scalar_norm_add, scalar_norm=scalar_norm, qk_norm_cache=qk_norm_cache,
     window_attention=window_attention, short_conv=short_conv, channel_delta=channel_delta,
@@ -1024,4 +1190,5 @@ ops = SimpleNamespace(expert_ffn=expert_ffn, ACT_GELU=ACT_GELU, ACT_RELU2=ACT_RE
     gate_mul=gate_mul, latent_rope_cache=latent_rope_cache, gla=gla, ACT_NONE=ACT_NONE, glu_rows=glu_rows,
     group_norm_add=group_norm_add, causal_conv=causal_conv, gated_delta=gated_delta, embed_stream=embed_stream,
     stream_split=stream_split, head_norm_cache=head_norm_cache, latent_down=latent_down, head_project=head_project,
-    ROUTER_SOFTMAX=ROUTER_SOFTMAX, ROUTER_SOFTMAX_CHOSEN=ROUTER_SOFTMAX_CHOSEN)
+    retention=retention, hyper_step=hyper_step, gated_act=gated_act, rope_operands=rope_operands, GATE_SILU=GATE_SILU,
+    GATE_GELU_TANH=GATE_GELU_TANH, ROUTER_SOFTMAX=ROUTER_SOFTMAX, ROUTER_SOFTMAX_CHOSEN=ROUTER_SOFTMAX_CHOSEN)

@@ -1,5 +1,6 @@
 """Configuration objects.  Field names follow vllm/config.py so engine arguments written
 for the reference (sep_prompt_token, kv_cache_dtype, block_size, quantization, ...) apply."""
+import importlib
 import json
 import os
 from typing import Optional
@@ -181,6 +182,36 @@ _DOVISUN_PRESETS = {
     "dovisun-2k": (2048, 2, 16, 4, 4224, 32, 2, 1408),   # up + down of 4224 = gate + up + down of 2816
     "dovisun-4k": (4096, 2, 32, 8, 8448, 32, 2, 2816),
 }
+
+
+def _vufasun_preset(width: int, passes: int, heads: int, kv_heads: int, ff: int, experts: int, top: int, expert_ff: int,
+                    shared_ff: int) -> dict:
+    """A Vufasun stack of layer sizes that resemble a served model's: four streams; a parallel layer (attention beside
+    retention), a block of two attention layers and a parallel layer that runs ``passes`` times, and three layers behind
+    it; dense feed-forwards and routed experts with a shared one in turn."""
+    d = width // heads
+    attn = {"heads": heads, "kv_heads": kv_heads, "dim": d, "vdim": d, "scale": d ** -0.5,
+            "rot": {"base": 500000.0, "dims": d // 2}}
+    left = dict(attn, rot={"base": 500000.0, "dims": d,
+                           "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}})
+    right = {"heads": heads // 2, "dim": d, "vdim": d, "rot": {"base": 10000.0, "dims": d},
+             "decay": [1.0 - 2.0 ** (-5 - 5 * i / max(heads // 2 - 1, 1)) for i in range(heads // 2)]}
+    par = {"left": left, "right": right}
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff}, "shared": {"ff": shared_ff}, "router": {"experts": experts, "top": top}}
+    kinds = [(par, dense), (attn, moe), (attn, dense), (par, moe), (attn, dense), (par, moe), (attn, None)]
+    layers = [{"type": "parallel" if m is par else "attention", "mixer": dict(m), "mlp": f} for m, f in kinds]
+    from .model_executor.models.vufasun import normalize_config
+    return normalize_config({"architecture": "Vufasun", "layers": layers, "loop": {"start": 1, "stop": 4, "times": passes},
+                             "norm": {"eps": 1e-6}, "streams": 4, "vocab": 32000, "width": width})
+
+
+_VUFASUN_PRESETS = {
+    # name: (width, passes of the block of three layers, heads, kv heads, feed-forward size, experts, top, expert ff, shared
+    # expert ff); two passes make ten layer runs; top 1 + shared = the active size of a top 2
+    "vufasun-2k": (2048, 2, 16, 4, 2816, 32, 1, 1408, 1408),
+    "vufasun-4k": (4096, 2, 32, 8, 5632, 32, 1, 2816, 2816),
+}
 # Llama stacks of the same width, depth and active feed-forward size, to measure the above against
 MODEL_PRESETS.update({
     "llama-2k": dict(architecture="llama", vocab_size=32000, hidden_size=2048, num_hidden_layers=10,
@@ -190,6 +221,9 @@ MODEL_PRESETS.update({
                      num_attention_heads=32, num_key_value_heads=8, intermediate_size=5632,
                      max_position_embeddings=8192, rms_norm_eps=1e-5, rope_theta=10000.0, torch_dtype="bfloat16"),
 })
+
+# decoders whose config.json lists their layers one by one: "architecture" names the module that reads it
+_LISTED_LAYER_MODELS = ("Nepevik", "Lapilorn", "Lalasun", "Bogetar", "Dovisun", "Vufasun")
 
 _ALIASES = {
     "facebook/opt-125m": "opt-125m", "meta-llama/Llama-2-7b-hf": "llama-2-7b",
@@ -247,25 +281,15 @@ class ModelConfig:
             return _bogetar_preset(*_BOGETAR_PRESETS[name])
         if name in _DOVISUN_PRESETS:
             return _dovisun_preset(*_DOVISUN_PRESETS[name])
+        if name in _VUFASUN_PRESETS:
+            return _vufasun_preset(*_VUFASUN_PRESETS[name])
         cfg_path = os.path.join(model, "config.json")
         if os.path.isfile(cfg_path):
             with open(cfg_path) as f:
                 raw = json.load(f)
-            if raw.get("architecture") == "Nepevik":
-                from .model_executor.models.nepevik import normalize_config
-                return normalize_config(raw)
-            if raw.get("architecture") == "Lapilorn":
-                from .model_executor.models.lapilorn import normalize_config
-                return normalize_config(raw)
-            if raw.get("architecture") == "Lalasun":
-                from .model_executor.models.lalasun import normalize_config
-                return normalize_config(raw)
-            if raw.get("architecture") == "Bogetar":
-                from .model_executor.models.bogetar import normalize_config
-                return normalize_config(raw)
-            if raw.get("architecture") == "Dovisun":
-                from .model_executor.models.dovisun import normalize_config
-                return normalize_config(raw)
+            if raw.get("architecture") in _LISTED_LAYER_MODELS:
+                module = importlib.import_module(f".model_executor.models.{raw['architecture'].lower()}", __package__)
+                return module.normalize_config(raw)
             arch = (raw.get("architectures") or [""])[0].lower()
             raw["architecture"] = "opt" if "opt" in arch else "llama"
             raw.setdefault("num_key_value_heads", raw["num_attention_heads"])

@@ -482,3 +482,61 @@ class LatentQueryAttention(nn.Module):
         _C.mixer_ops.capped_attention(mixed, q32, cache, None, None, md.ragged, H, 1, width, self.rank, self.scale)
         _C.mixer_ops.head_project(out.unflatten(1, (H, self.vdim)), mixed.unflatten(1, (H, self.rank)), self.value_up.data,
                                   gate=gate)
+
+
+class RotaryPagedAttention(nn.Module):
+    """Causal softmax attention with grouped query heads over a paged cache: rotary embedding on the pairs (i, i + rot / 2)
+    of the first rot coordinates (frequencies given as a table, angles from fp32 positions), score = (q . k) * scale;
+    optionally (``whole_norm_eps``) ONE RMS norm over all heads of the queries, and one over all heads of the keys, before
+    the rotation; optionally (``sink``) one more term exp(sink[head]) in the softmax's denominator, a learned number per
+    query head.  Keys are cached after norm and rotation; caches are [pages, page, kv_heads * size].  Norms, positions,
+    scores, weights and sums are fp32.
+
+    ``prepare`` and ``attend`` are the two halves of ``forward``: a layer that runs this attention beside a linear mixer on
+    the same projections has the operands of both prepared in one launch."""
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, inv_freq: torch.Tensor,
+                 whole_norm_eps: Optional[float] = None, sink: bool = False) -> None:
+        super().__init__()
+        if heads % kv_heads != 0:
+            raise ValueError(f"{heads} query heads cannot share {kv_heads} key/value heads evenly")
+        self.heads, self.kv_heads, self.dim, self.vdim, self.scale = heads, kv_heads, dim, vdim, float(scale)
+        if 2 * inv_freq.numel() > dim:
+            raise ValueError(f"{2 * inv_freq.numel()} rotated coordinates of heads of {dim}")
+        self.register_buffer("inv_freq", inv_freq.to(torch.float32).clone(), persistent=False)
+        self.norm_eps = whole_norm_eps
+        self.q_norm = self.k_norm = self.sink = None
+        if whole_norm_eps is not None:
+            self.q_norm = nn.Parameter(torch.ones(heads * dim, dtype=torch.float32), requires_grad=False)
+            self.k_norm = nn.Parameter(torch.ones(kv_heads * dim, dtype=torch.float32), requires_grad=False)
+        if sink:
+            self.sink = nn.Parameter(torch.zeros(heads, dtype=torch.float32), requires_grad=False)
+
+    def cache_shapes(self, block_size: int):
+        """Per page: keys, values."""
+        return [(block_size, self.kv_heads * self.dim), (block_size, self.kv_heads * self.vdim)]
+
+    def prepare(self, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, positions: torch.Tensor, key_cache: torch.Tensor,
+                value_cache: torch.Tensor, md: InputMetadata, linear: Optional[tuple] = None) -> torch.Tensor:
+        """q, k, v: column ranges of one projection output.  Fills the caches (and what ``linear`` names, the operands of a
+        linear mixer on the same projections); -> the queries, fp32 [rows, heads * dim]."""
+        q32 = torch.empty(q.shape[0], self.heads * self.dim, dtype=torch.float32, device=q.device)
+        normed = self.q_norm is not None
+        _C.mixer_ops.rope_operands(positions, (q32, q, k, v, self.inv_freq, self.heads, self.kv_heads, self.dim, self.vdim,
+                                               key_cache, value_cache, md.slot_mapping), linear,
+                                   self.q_norm.data if normed else None, self.k_norm.data if normed else None,
+                                   self.norm_eps if normed else 0.0)
+        return q32
+
+    def attend(self, q32: torch.Tensor, key_cache: torch.Tensor, value_cache: torch.Tensor, md: InputMetadata,
+               dtype: torch.dtype) -> torch.Tensor:
+        """-> [rows, heads * vdim]."""
+        out = torch.empty(q32.shape[0], self.heads * self.vdim, dtype=dtype, device=q32.device)
+        _C.mixer_ops.capped_attention(out, q32, key_cache, value_cache, None, md.ragged, self.heads, self.kv_heads, self.dim,
+                                      self.vdim, self.scale, sink=False if self.sink is None else self.sink.data)
+        return out
+
+    def forward(self, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, positions: torch.Tensor, key_cache: torch.Tensor,
+                value_cache: torch.Tensor, md: InputMetadata) -> torch.Tensor:
+        q32 = self.prepare(q, k, v, positions, key_cache, value_cache, md)
+        return self.attend(q32, key_cache, value_cache, md, q.dtype)

@@ -6,7 +6,7 @@ vllm/model_executor/layers/layernorm.py:10-65, rotary_embedding.py:36-141,
 activation.py:15-44.
 """
 import math
-from typing import Optional, Tuple, Union
+from typing import Dict, Optional, Tuple, Union
 
 import torch
 import torch.nn as nn
@@ -388,4 +388,64 @@ class ReluSquared(nn.Module):
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
         _C.mixer_ops.relu2(out, x)
+        return out
+
+
+class GatedActivation(nn.Module):
+    """x = gate | up -> act(gate) * up, act = silu or the tanh form of gelu (``kind``: "silu", "gelu_tanh")."""
+
+    def __init__(self, kind: str) -> None:
+        super().__init__()
+        self.kind = kind
+        self.code = {"silu": _C.mixer_ops.GATE_SILU, "gelu_tanh": _C.mixer_ops.GATE_GELU_TANH}[kind]
+
+    def _forward(self, x: torch.Tensor) -> torch.Tensor:
+        d = x.shape[-1] // 2
+        z = x[..., :d].float()
+        act = F.silu(z) if self.kind == "silu" else F.gelu(z, approximate="tanh")
+        return (act * x[..., d:].float()).to(x.dtype)
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        out = torch.empty(x.shape[0], x.shape[1] // 2, dtype=x.dtype, device=x.device)
+        _C.mixer_ops.gated_act(out, x, self.code)
+        return out
+
+
+class HyperConnection(nn.Module):
+    """How one sublayer is tied to a residual of several fp32 streams (hyper-connections): it reads
+    sum_j reads[j] x_j, and its output y goes back as x_j <- sum_i mix[i, j] x_i + writes[j] y, all streams at once from
+    the old ones (``mix`` is indexed [from, to]).  ``step`` is everything between this sublayer and the next one -- the
+    write, the next sublayer's read and its norm -- in one pass over the streams.  At a model's start the streams are all
+    equal to the embedding rows: ``begin`` and the first ``step`` take them from the embedding table (``origin``), so the
+    copies are never written."""
+
+    def __init__(self, streams: int) -> None:
+        super().__init__()
+        self.reads = nn.Parameter(torch.ones(streams, dtype=torch.float32), requires_grad=False)
+        self.writes = nn.Parameter(torch.ones(streams, dtype=torch.float32), requires_grad=False)
+        self.mix = nn.Parameter(torch.eye(streams, dtype=torch.float32), requires_grad=False)
+
+    def load_named(self, state: Dict[str, torch.Tensor], name: str) -> None:
+        """``state``: name.in, name.out, name.mix."""
+        self.reads.data.copy_(state[name + ".in"].float())
+        self.writes.data.copy_(state[name + ".out"].float())
+        self.mix.data.copy_(state[name + ".mix"].float())
+
+    @staticmethod
+    def begin(origin: Tuple[torch.Tensor, torch.Tensor], reads: torch.Tensor, norm: "OffsetRMSNorm") -> torch.Tensor:
+        """origin = (token ids, embedding table) -> what the first sublayer reads, normed, in the table's dtype."""
+        ids, table = origin
+        out = torch.empty(ids.numel(), table.shape[1], dtype=table.dtype, device=table.device)
+        _C.mixer_ops.hyper_step(None, out, norm.variance_epsilon, origin, reads=reads, weight=norm.weight.data)
+        return out
+
+    def step(self, streams: torch.Tensor, next_reads: torch.Tensor, next_norm: "OffsetRMSNorm", out_dtype: torch.dtype,
+             a: Optional[torch.Tensor] = None, b: Optional[torch.Tensor] = None, c: Optional[torch.Tensor] = None,
+             norms: Optional[Tuple[torch.Tensor, torch.Tensor]] = None, blend: float = 1.0,
+             origin: Optional[Tuple[torch.Tensor, torch.Tensor]] = None) -> torch.Tensor:
+        """streams fp32 [rows, S, width], in place; the sublayer's output is a + b + c (c fp32), or with ``norms``
+        blend * (N(a) + N(b)), the two RMS norms' weights given.  -> what the next sublayer reads, normed."""
+        out = torch.empty(streams.shape[0], streams.shape[2], dtype=out_dtype, device=streams.device)
+        _C.mixer_ops.hyper_step(streams, out, next_norm.variance_epsilon, origin, self.mix.data, self.writes.data, a, b, c,
+                                norms, blend, next_reads, next_norm.weight.data)
         return out

@@ -13,6 +13,9 @@ routed sum so that the caller's residual add can take both.  The same layer, by 
 a gated hidden layer with limits (``activation="clamped_glu"``: g = min(gate x, limit), u = clamp(up x, +-limit),
 g sigmoid(alpha g) (u + shift); alpha 1, no limit and shift 0 make it silu(g) u).  ``score="softmax_chosen"``: the choice
 goes by the logits and the weights are their softmax over the chosen ones (a ``router_bias`` is part of the logits).
+``weigh_input``: an expert's weight multiplies what the expert reads instead of what it returns (the two differ: the
+hidden layer is not linear).  A shared expert has the routed experts' form: with a gated hidden layer it is
+down(silu(gate x) * up x).
 
 Rows are grouped by expert on the device (a stable sort of the (row, choice) pairs by expert id, then a binary
 search for every expert's first pair), so each expert's rows are one contiguous run and the host never waits.
@@ -24,6 +27,7 @@ import torch.nn as nn
 import torch.nn.functional as F
 
 from ... import _C
+from .basic import GatedActivation, ReluSquared
 from .linear import ColumnParallelLinear, MergedColumnParallelLinear, RowParallelLinear
 
 
@@ -84,13 +88,14 @@ class GroupRoutedExperts(nn.Module):
                  keep_groups: int, scale: float, dtype: torch.dtype, linear_method=None, score: str = "sigmoid",
                  group_score: str = "top2", normalize: bool = True, activation: str = "relu2",
                  limit: float = float("inf"), glu_alpha: float = 1.702, glu_shift: float = 1.0, router_bias: bool = False,
-                 router_dtype: torch.dtype = torch.float32) -> None:
+                 router_dtype: torch.dtype = torch.float32, weigh_input: bool = False) -> None:
         super().__init__()
         if score not in ("sigmoid", "softmax", "softmax_chosen") or group_score not in ("top2", "max") or \
                 activation not in ("relu2", "clamped_glu"):
             raise ValueError(f"unknown router score {score!r}, group score {group_score!r} or activation {activation!r}")
-        if activation == "clamped_glu" and shared_ff:
-            raise NotImplementedError("a shared expert with a gated hidden layer")
+        if activation == "clamped_glu" and shared_ff and (glu_alpha, limit, glu_shift) != (1.0, float("inf"), 0.0):
+            raise NotImplementedError("a shared expert whose gated hidden layer is not silu(gate) * up")
+        self.weigh_input = bool(weigh_input)
         self.softmax = {"sigmoid": 0, "softmax": _C.mixer_ops.ROUTER_SOFTMAX,
                         "softmax_chosen": _C.mixer_ops.ROUTER_SOFTMAX_CHOSEN}[score]
         self.group_best_one, self.normalize = group_score == "max", bool(normalize)
@@ -111,7 +116,9 @@ class GroupRoutedExperts(nn.Module):
         self.down = nn.Parameter(torch.empty(num_experts, width, ff, dtype=dtype), requires_grad=False)
         self.shared_ff = shared_ff
         if shared_ff:
-            self.shared_up = ColumnParallelLinear(width, shared_ff, False, dtype, linear_method)
+            self.shared_up = MergedColumnParallelLinear(width, [shared_ff, shared_ff], False, dtype, linear_method) \
+                if self.glu else ColumnParallelLinear(width, shared_ff, False, dtype, linear_method)
+            self.shared_act = GatedActivation("silu") if self.glu else ReluSquared()
             self.shared_down = RowParallelLinear(shared_ff, width, False, dtype, linear_method)
 
     def router_logits(self, h: torch.Tensor) -> torch.Tensor:
@@ -134,13 +141,11 @@ class GroupRoutedExperts(nn.Module):
                                                     self.normalize, clear=out)
         order, start = group_pairs_by_expert(chosen, self.num_experts)
         _C.mixer_ops.expert_ffn(out, h, self.up.data, self.down.data, order, start, self.top, 1.0,
-                                activation=_C.mixer_ops.ACT_RELU2, pair_weight=weights, glu=self.glu)
+                                activation=_C.mixer_ops.ACT_RELU2, pair_weight=weights, glu=self.glu,
+                                weigh_input=self.weigh_input)
         shared = None
         if self.shared_ff:
-            hidden = self.shared_up(h)
-            act = torch.empty_like(hidden)
-            _C.mixer_ops.relu2(act, hidden)
-            shared = self.shared_down(act)
+            shared = self.shared_down(self.shared_act(self.shared_up(h)))
         return shared, out
 
     def load_named(self, w: Dict[str, torch.Tensor]) -> None:
@@ -156,5 +161,5 @@ class GroupRoutedExperts(nn.Module):
             self.up.data.copy_(torch.stack([w[f"e{e}.up"] for e in range(self.num_experts)]))
         self.down.data.copy_(torch.stack([w[f"e{e}.down"] for e in range(self.num_experts)]))
         if self.shared_ff:
-            self.shared_up.weight.data.copy_(w["shared.up"])
+            self.shared_up.weight.data.copy_(torch.cat([w["shared.gate"], w["shared.up"]], 0) if self.glu else w["shared.up"])
             self.shared_down.weight.data.copy_(w["shared.down"])

@@ -20,6 +20,8 @@ Linear attention, per head, S [key size, value size]:
   ``GatedLinearAttentionMixer``  S <- diag(a) S + k v^T;  o = S^T q dim^(-1/2),  a = sigmoid(low-rank(h) + b)^(1 / tau)
                           per head and key channel; each head's output is normed with a weight shared by the
                           heads, gated by silu(gate) and projected
+  ``RetentionMixer``      S <- decay_h S + k v^T;  o = S^T q,  q and k rotated by their position, k times dim^(-1/2);
+                          each head's output is divided by its root mean square and gated by silu(gate)
 """
 from typing import Dict, List, Sequence, Tuple
 
@@ -282,3 +284,46 @@ class GatedLinearAttentionMixer(nn.Module):
         self.decay_up.weight.data.copy_(w["a2"])
         self.decay_bias.data.copy_(w["a2.b"].float())
         self.out_norm.data.copy_(w["norm"].float())
+
+
+class RetentionMixer(nn.Module):
+    """Linear attention with one constant decay per head on rotated queries and keys (pairs (i, i + rot / 2), angles from
+    fp32 positions; the keys also times dim^-1/2), no softmax and no denominator; each head's output is divided by its root
+    mean square (no weight) and gated by silu(gate).  The mixer owns no projections: its layer hands over column ranges
+    of its input GEMM and projects the result.  Queries, keys, recurrence, state and norm are fp32."""
+
+    def __init__(self, heads: int, dim: int, vdim: int, decay: Sequence[float], inv_freq: torch.Tensor, eps: float) -> None:
+        super().__init__()
+        if len(decay) != heads or 2 * inv_freq.numel() > dim:
+            raise ValueError(f"retention: {len(decay)} decays and {2 * inv_freq.numel()} rotated coordinates for {heads} "
+                             f"heads of {dim}")
+        self.heads, self.dim, self.vdim, self.eps = heads, dim, vdim, eps
+        # constants of the config, not weights
+        self.register_buffer("decay", torch.tensor([float(d) for d in decay], dtype=torch.float64).to(torch.float32),
+                             persistent=False)
+        self.register_buffer("inv_freq", inv_freq.to(torch.float32).clone(), persistent=False)
+
+    def state_shapes(self) -> List[Tuple[int, ...]]:
+        return [(self.heads, self.dim, self.vdim)]
+
+    def operands(self, q: torch.Tensor, k: torch.Tensor) -> tuple:
+        """What ``mixer_ops.rope_operands`` takes as its linear side; its first two entries are the fp32 results."""
+        new = lambda: torch.empty(q.shape, dtype=torch.float32, device=q.device)        # noqa: E731
+        return (new(), new(), q, k, self.inv_freq, self.heads, self.dim, self.dim ** -0.5)
+
+    def core(self, q32: torch.Tensor, k32: torch.Tensor, v: torch.Tensor, gate: torch.Tensor, state: torch.Tensor,
+             md: InputMetadata) -> torch.Tensor:
+        """q32, k32: prepared operands; v, gate: column ranges of the projection output.  -> the normed, gated heads
+        [rows, heads * vdim], before the output projection."""
+        rows, nv = v.shape[0], self.heads * self.vdim
+        o = torch.empty(rows, nv, dtype=torch.float32, device=v.device)
+        _C.mixer_ops.retention(o, q32, k32, v, self.decay, state, md.ragged, self.heads, self.dim, self.vdim)
+        gated = torch.empty(rows, nv, dtype=v.dtype, device=v.device)
+        _C.mixer_ops.head_norm_gate(gated, o, gate, None, False, self.eps, self.heads, self.vdim, gate_silu=True)
+        return gated
+
+    def forward(self, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor, positions: torch.Tensor,
+                state: torch.Tensor, md: InputMetadata) -> torch.Tensor:
+        ready = self.operands(q, k)
+        _C.mixer_ops.rope_operands(positions, linear=ready)
+        return self.core(ready[0], ready[1], v, gate, state, md)

@@ -20,10 +20,11 @@ from .models.lapilorn import LapilornForCausalLM
 from .models.llama import LlamaForCausalLM
 from .models.nepevik import NepevikForCausalLM
 from .models.opt import OPTForCausalLM
+from .models.vufasun import VufasunForCausalLM
 
 _ARCH = {"llama": LlamaForCausalLM, "opt": OPTForCausalLM, "nepevik": NepevikForCausalLM,
          "lapilorn": LapilornForCausalLM, "lalasun": LalasunForCausalLM, "bogetar": BogetarForCausalLM,
-         "dovisun": DovisunForCausalLM}
+         "dovisun": DovisunForCausalLM, "vufasun": VufasunForCausalLM}
 
 
 def architecture_class(name: str):

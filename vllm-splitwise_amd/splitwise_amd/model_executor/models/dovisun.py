@@ -21,7 +21,7 @@ Steps arrive in the ragged layout (``InputMetadata.ragged``): any mix of prompt 
 The worker allocates what ``cache_layout`` asks for per layer RUN: a layer that runs several times has pages of its own
 for every pass.
 """
-from typing import Dict, List, Optional, Tuple
+from typing import Dict, List, Optional
 
 import torch
 import torch.nn as nn
@@ -35,6 +35,7 @@ from ..layers.moe import GroupRoutedExperts
 from ..layers.sampler import Sampler, SamplingMetadata
 from ..layers.vocab_parallel_embedding import VocabParallelEmbedding
 from ..parallel_state import get_tensor_model_parallel_world_size
+from .layer_list import layer_runs
 
 _MIXERS = ("attention", "latent_attention")
 _DEFAULT_Q_RANK_DIVISOR = 4       # of a model without a checkpoint whose config does not name the query latent's size
@@ -53,20 +54,6 @@ def normalize_config(raw: dict) -> dict:
     cfg.setdefault("max_position_embeddings", 1 << 20)       # angles come from fp32 positions: no table to outgrow
     cfg.setdefault("torch_dtype", "bfloat16")
     return cfg
-
-
-def layer_runs(cfg: dict) -> List[Tuple[int, bool]]:
-    """[(layer, does a pass of the loop begin here?)] in the order the layers run."""
-    n, loop = len(cfg["layers"]), cfg.get("loop")
-    if not loop:
-        return [(i, False) for i in range(n)]
-    start, stop, times = int(loop["start"]), int(loop["stop"]), int(loop["times"])
-    if not (0 <= start < stop <= n) or times < 1:
-        raise ValueError(f"loop over layers {start} .. {stop - 1}, {times} times, of a model of {n} layers")
-    runs = [(i, False) for i in range(start)]
-    for _ in range(times):
-        runs += [(i, i == start) for i in range(start, stop)]
-    return runs + [(i, False) for i in range(stop, n)]
 
 
 def _q_rank(cfg: dict, m: dict) -> int:
