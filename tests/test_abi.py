@@ -50,3 +50,23 @@ def test_argument_errors_are_reported_without_a_gpu():
     rc = lib.sw_convert_fp8_e5m2(None, None, 8, _C.SW_F16, _C.SW_F16, None)
     assert rc == -1
     assert b"fp8" in lib.sw_last_error()
+
+
+def test_mixers_binding_matches_its_header():
+    """Every signature of the mixer binding, argument by argument, against the header's declaration."""
+    from splitwise_amd import _C_mixers as m
+    header = re.sub(r"/\*.*?\*/", "", open(os.path.join(ROOT, "include", "splitwise_mixers.h")).read(), flags=re.S)
+    assert int(re.search(r"#define SWM_ABI_VERSION (\d+)", header).group(1)) == m.ABI_VERSION
+    kind = {m._p: "pointer", m._l: "int64", m._f: "float", m._i: "int"}
+    for name, signature in m._SIGNATURES.items():
+        args = re.search(r"\bint " + name + r"\(([^;]*)\);", header).group(1).split(",")
+        declared = ["pointer" if "*" in a else "int64" if "int64_t" in a else "float" if "float" in a else "int" for a in args]
+        assert [kind[t] for t in signature] == declared, name
+
+
+@pytest.mark.skipif(not os.path.exists(os.path.join(PKG, "splitwise_amd", "libsplitwise_mixers.so")), reason="library not built")
+def test_mixers_library_exports_what_the_binding_names():
+    from splitwise_amd import _C_mixers
+    lib = _C_mixers.load_library()
+    for name in _C_mixers._SIGNATURES:
+        assert hasattr(lib, name), name

@@ -1,4 +1,4 @@
-"""Throughput of a Nepevik (or Lapilorn, Lalasun, Bogetar or Dovisun) stack beside a Llama stack of the same width, depth and active feed-forward size
+"""Throughput of a Nepevik (or Lapilorn, Lalasun, Bogetar, Dovisun or Vufasun) stack beside a Llama stack of the same width, depth and active feed-forward size
 (random weights), and every mixer kernel beside the like kernel of the Llama path with their distances from
 the roofline.  ``bench.py --mixers`` prints the result as one JSON line.
 
@@ -832,8 +832,143 @@ def kernel_table_dovisun(width: int = 2048, heads: int = 16, kv_heads: int = 4, 
     return rows
 
 
+@torch.inference_mode()
+def kernel_table_vufasun(width: int = 2048, heads: int = 16, kv_heads: int = 4, prefill_rows: int = 4096,
+                         decode_seqs: int = 64, decode_ctx: int = 2047, streams: int = 4, ff: int = 2816, experts: int = 32,
+                         top: int = 1, expert_ff: int = 1408) -> List[dict]:
+    """The kernels of the Vufasun layers beside their like: attention with a learned sink beside Dovisun's sink of exp(0);
+    the rotated operands of one mixer and of two beside the rotation kernel of Lapilorn and Bogetar (with a norm per head);
+    retention beside lightning attention, with their output norms; the step of the streams in its four forms beside the
+    fused add + norm of one stream (Dovisun) and the one behind a norm (Bogetar); the gated activation, the router and the
+    experts beside theirs."""
+    from .. import _C
+    ops = _C.mixer_ops
+    dev, bf = torch.device("cuda"), torch.bfloat16
+    d, page, S = width // heads, 16, streams
+    r_heads = heads // 2
+    rows: List[dict] = []
+    for phase, seqs in (("prefill", [(0, prefill_rows // 2, 0, None), (0, prefill_rows // 2, 1, None)]),
+                        ("decode", [(decode_ctx, 1, i, None) for i in range(decode_seqs)])):
+        total_pages, laid = 0, []
+        for ctx, n, slot, _ in seqs:
+            pages = -(-(ctx + n) // page)
+            laid.append((ctx, n, slot, list(range(total_pages, total_pages + pages))))
+            total_pages += pages
+        batch = _ragged(laid, dev)
+        T, B = sum(s[1] for s in laid), len(laid)
+        lbatch = _ragged([(c, n, i, []) for i, (c, n, _, _) in enumerate(laid)], dev)
+        pairs = sum(i + 1 for c, n, _, _ in laid for i in range(c, c + n))
+        keys = sum(c + n for c, n, _, _ in laid)
+        pos = torch.cat([torch.arange(c, c + n) for c, n, _, _ in laid]).to(dev)
+        slots = torch.cat([torch.tensor([tb[p // page] * page + p % page for p in range(c, c + n)])
+                           for c, n, _, tb in laid]).to(dev)
+        # ---------------------------------------------------------------- attention
+        kc = torch.randn(total_pages, page, kv_heads * d, device=dev).to(bf)
+        vc = torch.randn(total_pages, page, kv_heads * d, device=dev).to(bf)
+        q, out = torch.randn(T, heads * d, device=dev), torch.empty(T, heads * d, dtype=bf, device=dev)
+        abytes = keys * kv_heads * d * 2 * 2 + T * heads * d * (4 + 2)
+        for name, sink, like in (("attention with a learned sink per head", torch.randn(heads, device=dev), ""),
+                                 ("Dovisun attention with a sink of exp(0)", True, "attention with a learned sink")):
+            t = _time(lambda: ops.capped_attention(out, q, kc, vc, None, batch, heads, kv_heads, d, d, d ** -0.5, sink=sink))
+            rows.append(_row(name, phase, t, abytes, 4.0 * pairs * heads * d, VALU_F32, like=like))
+        # ---------------------------------------------------------------- rotated operands
+        rd = r_heads * d
+        sizes = [heads * d, kv_heads * d, kv_heads * d, rd, rd, rd, rd]
+        proj = torch.randn(T, sum(sizes), device=dev).to(bf)
+        qc, kcol, vcol, rq, rk, rv, gate = proj.split(sizes, 1)
+        q32, lq, lk = torch.empty(T, heads * d, device=dev), torch.empty(T, rd, device=dev), torch.empty(T, rd, device=dev)
+        inv = torch.rand(d // 2, device=dev)
+        wq, wk, wd = torch.ones(heads * d, device=dev), torch.ones(kv_heads * d, device=dev), torch.ones(d, device=dev)
+        att = (q32, qc, kcol, vcol, inv, heads, kv_heads, d, d, kc, vc, slots)
+        nbytes = T * ((heads + 2 * kv_heads) * d * 2 + heads * d * 4 + 2 * kv_heads * d * 2)
+        lbytes = T * rd * 2 * (2 + 4)
+        t = _time(lambda: ops.rope_operands(pos, att))
+        rows.append(_row("rope_operands (attention)", phase, t, nbytes, 6.0 * T * heads * d, VALU_F32))
+        t = _time(lambda: ops.rope_cache(q32, qc, kcol, vcol, pos, inv, heads, kv_heads, d, d, kc, vc, slots, True))
+        rows.append(_row("Lapilorn rope_cache", phase, t, nbytes, 6.0 * T * heads * d, VALU_F32, like="rope_operands"))
+        t = _time(lambda: ops.rope_operands(pos, att, (lq, lk, rq, rk, inv, r_heads, d, d ** -0.5), wq, wk, 1e-6))
+        rows.append(_row("rope_operands (whole-projection norm, retention's operands in the same launch)", phase, t,
+                         nbytes + lbytes, 6.0 * T * (heads * d + 2 * rd), VALU_F32))
+        t = _time(lambda: ops.rope_cache(q32, qc, kcol, vcol, pos, inv, heads, kv_heads, d, d, kc, vc, slots, True, wd, wd, 1e-6))
+        rows.append(_row("Bogetar rope_cache behind a per-head norm (attention's operands only)", phase, t, nbytes,
+                         10.0 * T * heads * d, VALU_F32, like="rope_operands"))
+        # ---------------------------------------------------------------- retention
+        state = torch.zeros(max(B, 2), r_heads, d, d, device=dev)
+        decay = torch.full((r_heads,), 0.97, device=dev)
+        o = torch.empty(T, rd, device=dev)
+        lflops = T * r_heads * (2.0 * 32 * d + 2.0 * 32 * d + 4.0 * d * d)
+        sbytes = 2 * B * r_heads * d * d * 4
+        t = _time(lambda: ops.retention(o, lq, lk, rv, decay, state, lbatch, r_heads, d, d))
+        rows.append(_row("retention (chunks of 32 on fp32 matrix cores)", phase, t, T * rd * (2 * 4 + 2 + 4) + sbytes, lflops, VALU_F32))
+        t = _time(lambda: ops.lightning(o, rq, rk, rv, decay, state, lbatch, r_heads, d, d))
+        rows.append(_row("Lapilorn lightning", phase, t, T * rd * (3 * 2 + 4) + sbytes, lflops, VALU_F32, like="retention"))
+        gated = torch.empty(T, rd, dtype=bf, device=dev)
+        for name, w, like in (("head_norm_gate (no weight, silu gate)", None, ""),
+                              ("Bogetar head_norm_gate (one weight for all heads, silu gate)", wd, "head_norm_gate")):
+            t = _time(lambda: ops.head_norm_gate(gated, o, gate, w, False, 1e-6, r_heads, d, gate_silu=True))
+            rows.append(_row(name, phase, t, T * rd * (4 + 2 + 2), 6.0 * T * rd, VALU_F32, like=like))
+        # ---------------------------------------------------------------- the streams
+        x, h = torch.randn(T, S, width, device=dev), torch.empty(T, width, dtype=bf, device=dev)
+        mix, writes, reads = 0.9 * torch.eye(S, device=dev) + 0.02, torch.ones(S, device=dev), torch.full((S,), 0.25, device=dev)
+        y1, y2, c32 = torch.randn(T, width, device=dev).to(bf), torch.randn(T, width, device=dev).to(bf), torch.randn(T, width, device=dev)
+        w, wa, wb = (torch.ones(width, device=dev) for _ in range(3))
+        table, ids = torch.randn(32000, width, device=dev).to(bf), torch.randint(0, 32000, (T,), device=dev)
+        wflops = T * width * (2.0 * S * S + 6.0 * S)
+
+        def hyper(name, extra, **kw):
+            origin = kw.pop("origin", None)
+            t = _time(lambda: ops.hyper_step(x, h, 1e-6, origin, mix, writes, reads=reads, weight=w, **kw))
+            moved = (0 if origin else S * 4) + S * 4 + 2 + extra
+            rows.append(_row(name, phase, t, T * width * moved, wflops, VALU_F32))
+        hyper("hyper_step (four streams, one addend, next norm)", 2, a=y1)
+        hyper("hyper_step (two addends, one fp32)", 2 + 4, a=y1, c=c32)
+        hyper("hyper_step (mean of two normed outputs)", 2 + 2, a=y1, b=y2, norms=(wa, wb), blend=0.5)
+        hyper("hyper_step (first write: old streams from the embedding table)", 2 + 2, a=y1, origin=(ids, table))
+        t = _time(lambda: ops.hyper_step(None, h, 1e-6, (ids, table), reads=reads, weight=w))
+        rows.append(_row("hyper_step (first read, from the embedding table)", phase, t, T * width * (2 + 2), 4.0 * T * width, VALU_F32))
+        stream = torch.randn(T, width, device=dev)
+        t = _time(lambda: ops.stream_add_norm(stream, w, 0.0, 1e-6, h, y1, None, c32))
+        rows.append(_row("Dovisun stream_add_norm (one stream, two addends, one fp32)", phase, t, T * width * (4 + 4 + 2 + 4 + 2),
+                         6.0 * T * width, VALU_F32, like="hyper_step"))
+        t = _time(lambda: ops.group_norm_add(stream, 8, 1e-6, y1, wa, None, y2, 0.8, 0.5, w, h))
+        rows.append(_row("Bogetar group_norm_add (one stream, a normed sum of two)", phase, t, T * width * (4 + 4 + 2 + 2 + 2),
+                         10.0 * T * width, VALU_F32, like="hyper_step"))
+        raw = torch.empty(T, width, dtype=bf, device=dev)
+        t = _time(lambda: ops.embed_stream(stream, ids, table, 1.0, raw, w, 0.0, 1e-6, h))
+        rows.append(_row("Dovisun embed_stream", phase, t, T * width * (2 + 4 + 2 + 2), 4.0 * T * width, VALU_F32, like="hyper_step (first)"))
+        # ---------------------------------------------------------------- feed-forward
+        gu, act = torch.randn(T, 2 * ff, device=dev).to(bf), torch.empty(T, ff, dtype=bf, device=dev)
+        for name, kind in (("gated_act (gelu, tanh form)", ops.GATE_GELU_TANH), ("gated_act (silu)", ops.GATE_SILU)):
+            t = _time(lambda: ops.gated_act(act, gu, kind))
+            rows.append(_row(name, phase, t, T * ff * 3 * 2, 10.0 * T * ff, VALU_F32))
+        t = _time(lambda: ops.clamped_glu(act, gu, 1.702, 7.0, 1.0))
+        rows.append(_row("Lapilorn clamped_glu", phase, t, T * ff * 3 * 2, 8.0 * T * ff, VALU_F32, like="gated_act"))
+        xin = torch.randn(T, width, device=dev).to(bf)
+        r16, eo = (torch.randn(experts, width, device=dev) * width ** -0.5).to(bf), torch.empty(T, width, device=dev)
+
+        def route(softmax, normalize):
+            return ops.group_router(torch.mm(xin, r16.t(), out_dtype=torch.float32), None, top, 1, 1, 1.0, softmax, False, normalize,
+                                    clear=eo)
+        rbytes = T * width * (2 + 4) + experts * width * 2 + T * top * 8
+        for name, args, like in (("router: sigmoid scores as they are", (0, False), ""),
+                                 ("Dovisun router: softmax over the chosen", (ops.ROUTER_SOFTMAX_CHOSEN, True), "router")):
+            t = _time(lambda: route(*args))
+            rows.append(_row(name, phase, t, rbytes, 2.0 * T * experts * width, VALU_F32, like=like))
+        chosen, weights = route(0, False)
+        order, start = ops.group_pairs(chosen, experts)
+        up = (torch.randn(experts, 32 * (-(-expert_ff // 16)), width, device=dev) * 0.02).to(bf)
+        down = (torch.randn(experts, width, expert_ff, device=dev) * 0.02).to(bf)
+        active = int((torch.bincount(chosen.flatten(), minlength=experts) > 0).sum())
+        ebytes = active * 3 * expert_ff * width * 2 + T * width * (2 + 4) + T * top * expert_ff * 2 * 2
+        for name, inp, like in (("expert_ffn (weight on the input)", True, ""), ("Dovisun expert_ffn (weight on the output)", False, "expert_ffn")):
+            t = _time(lambda: ops.expert_ffn(eo, xin, up, down, order, start, top, 1.0, pair_weight=weights,
+                                             glu=(1.0, float("inf"), 0.0), weigh_input=inp))
+            rows.append(_row(name, phase, t, ebytes, 6.0 * T * top * expert_ff * width, MFMA_BF16, like=like))
+    return rows
+
+
 # the existing families that a stack is measured beside
-_BESIDE = {"dovisun": ("lalasun", "bogetar", "llama")}
+_BESIDE = {"dovisun": ("lalasun", "bogetar", "llama"), "vufasun": ("dovisun", "bogetar", "llama")}
 
 
 def run(sizes=("2k",), with_kernels: bool = True, family: str = "nepevik") -> dict:
@@ -845,6 +980,6 @@ def run(sizes=("2k",), with_kernels: bool = True, family: str = "nepevik") -> di
         result["engine"][size] = pair
     if with_kernels:
         table = {"nepevik": kernel_table, "lapilorn": kernel_table_lapilorn, "lalasun": kernel_table_lalasun,
-                 "bogetar": kernel_table_bogetar, "dovisun": kernel_table_dovisun}[family]
+                 "bogetar": kernel_table_bogetar, "dovisun": kernel_table_dovisun, "vufasun": kernel_table_vufasun}[family]
         result["kernels"]["2k"] = table()
     return result
