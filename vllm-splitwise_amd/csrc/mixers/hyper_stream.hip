@@ -15,25 +15,6 @@ namespace swm {
 constexpr int kMaxStreams = 8;
 constexpr int kHyperMaxThreads = 1024;
 
-// V neighbouring numbers of type T, widened
-template <typename T, int V>
-__device__ __forceinline__ void ld_vec(float (&x)[V], const void* p, int64_t i) {
-  using S = typename Conv<T>::store_t;
-  struct alignas(V * sizeof(S)) Piece { S e[V]; };
-  const Piece q = *reinterpret_cast<const Piece*>(static_cast<const S*>(p) + i);
-#pragma unroll
-  for (int j = 0; j < V; ++j) x[j] = Conv<T>::to_float(q.e[j]);
-}
-template <typename T, int V>
-__device__ __forceinline__ void st_vec(void* p, int64_t i, const float (&x)[V]) {
-  using S = typename Conv<T>::store_t;
-  struct alignas(V * sizeof(S)) Piece { S e[V]; };
-  Piece q;
-#pragma unroll
-  for (int j = 0; j < V; ++j) q.e[j] = Conv<T>::from_float(x[j]);
-  *reinterpret_cast<Piece*>(static_cast<S*>(p) + i) = q;
-}
-
 struct HyperArgs {
   float* streams;              // [rows, S, width]
   const int64_t* ids;          // not NULL: every old stream of a row is table[ids[row]]

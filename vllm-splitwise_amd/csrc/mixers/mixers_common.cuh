@@ -20,6 +20,25 @@ __device__ __forceinline__ void st(void* p, int64_t i, float v) {
   static_cast<typename Conv<T>::store_t*>(p)[i] = Conv<T>::from_float(v);
 }
 
+// V neighbouring numbers of type T, widened
+template <typename T, int V>
+__device__ __forceinline__ void ld_vec(float (&x)[V], const void* p, int64_t i) {
+  using S = typename Conv<T>::store_t;
+  struct alignas(V * sizeof(S)) Piece { S e[V]; };
+  const Piece q = *reinterpret_cast<const Piece*>(static_cast<const S*>(p) + i);
+#pragma unroll
+  for (int j = 0; j < V; ++j) x[j] = Conv<T>::to_float(q.e[j]);
+}
+template <typename T, int V>
+__device__ __forceinline__ void st_vec(void* p, int64_t i, const float (&x)[V]) {
+  using S = typename Conv<T>::store_t;
+  struct alignas(V * sizeof(S)) Piece { S e[V]; };
+  Piece q;
+#pragma unroll
+  for (int j = 0; j < V; ++j) q.e[j] = Conv<T>::from_float(x[j]);
+  *reinterpret_cast<Piece*>(static_cast<S*>(p) + i) = q;
+}
+
 __device__ __forceinline__ float sigmoidf_(float x) { return 1.0f / (1.0f + expf(-x)); }
 // softplus without overflow: log(1 + e^x) = max(x, 0) + log1p(e^-|x|)
 __device__ __forceinline__ float softplusf_(float x) { return fmaxf(x, 0.0f) + log1pf(expf(-fabsf(x))); }

@@ -24,25 +24,7 @@ struct RopeSide {
   void* v_out;                 // attention: the value cache
 };
 
-// V neighbours per access (1: any sizes and strides)
-template <typename T, int V>
-struct RopePiece {
-  using S = typename Conv<T>::store_t;
-  struct alignas(V * sizeof(S)) P { S e[V]; };
-  static __device__ __forceinline__ void load(float (&x)[V], const void* p, int64_t i) {
-    const P q = *reinterpret_cast<const P*>(static_cast<const S*>(p) + i);
-#pragma unroll
-    for (int j = 0; j < V; ++j) x[j] = Conv<T>::to_float(q.e[j]);
-  }
-  static __device__ __forceinline__ void store(void* p, int64_t i, const float (&x)[V]) {
-    P q;
-#pragma unroll
-    for (int j = 0; j < V; ++j) q.e[j] = Conv<T>::from_float(x[j]);
-    *reinterpret_cast<P*>(static_cast<S*>(p) + i) = q;
-  }
-};
-
-// the heads at src[off ..] turned: dst[dst_off ..] = scale * rotate(x * fac * norm)
+// V: neighbours per access (1: any sizes and strides).  The heads at src[off ..] turned: dst[dst_off ..] = scale * rotate(x * fac * norm)
 template <typename T, typename TO, int V>
 __device__ __forceinline__ void turn_heads(void* __restrict__ dst, int64_t dst_off, const void* __restrict__ src, int64_t off,
                                            int heads, int dim, int half, float fac, const float* __restrict__ norm,
@@ -53,8 +35,8 @@ __device__ __forceinline__ void turn_heads(void* __restrict__ dst, int64_t dst_o
     float a[V];
     if (i < half) {
       float b[V];
-      RopePiece<T, V>::load(a, src, off + base + i);
-      RopePiece<T, V>::load(b, src, off + base + i + half);
+      ld_vec<T, V>(a, src, off + base + i);
+      ld_vec<T, V>(b, src, off + base + i + half);
       if (norm != nullptr) {
 #pragma unroll
         for (int j = 0; j < V; ++j) {
@@ -68,13 +50,13 @@ __device__ __forceinline__ void turn_heads(void* __restrict__ dst, int64_t dst_o
         a[j] = (u * c - w * s) * scale;
         b[j] = (w * c + u * s) * scale;
       }
-      RopePiece<TO, V>::store(dst, dst_off + base + i, a);
-      RopePiece<TO, V>::store(dst, dst_off + base + i + half, b);
+      st_vec<TO, V>(dst, dst_off + base + i, a);
+      st_vec<TO, V>(dst, dst_off + base + i + half, b);
     } else {
-      RopePiece<T, V>::load(a, src, off + base + i + half);
+      ld_vec<T, V>(a, src, off + base + i + half);
 #pragma unroll
       for (int j = 0; j < V; ++j) a[j] *= (norm != nullptr ? fac * norm[base + i + half + j] : 1.0f) * scale;
-      RopePiece<TO, V>::store(dst, dst_off + base + i + half, a);
+      st_vec<TO, V>(dst, dst_off + base + i + half, a);
     }
   }
 }
